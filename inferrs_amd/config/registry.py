@@ -24,6 +24,7 @@ from .ligizen import LigizenConfig
 from .lofudra import LofudraConfig
 from .qwen3 import Qwen3Config
 from .spec import ModelSpec
+from .vufizen import VufizenConfig
 
 _BY_ARCHITECTURE: Dict[str, Type] = {}
 _BY_MODEL_TYPE: Dict[str, Type] = {}
@@ -76,3 +77,4 @@ register_architecture(BuketarConfig)
 register_architecture(LofudraConfig)
 register_architecture(FisanexConfig)
 register_architecture(LigizenConfig)
+register_architecture(VufizenConfig)

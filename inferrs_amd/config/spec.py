@@ -28,6 +28,7 @@ class NormSpec:
     eps: float
     add_one: bool = False          # weight is stored as (w - 1) when True
     kind: str = "rmsnorm"
+    scalar: bool = False           # the file holds ONE number (a tensor of shape []) that weighs every feature
 
 
 @dataclass(frozen=True)
@@ -231,6 +232,40 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class DifferentialAttentionSpec:
+    """Softmax attention of two maps a head over shared values, the second taken off the first: q is n_heads * 2 *
+    head_dim rows and k n_kv_heads * 2 * head_dim, head by head [map 1 | map 2]; lambda = exp(lq1 . lk1) - exp(lq2 . lk2) +
+    `diff`, one number a layer; o = a1 - lambda a2, brought to unit root mean square a head (`norm_eps`), times 1 -
+    `diff`.  Ahead of the maps q, k and v pass a causal convolution of `conv` taps a channel (tensors "q.conv", "k.conv",
+    "v.conv" [channels, conv], no bias), q and k then an RMS norm a map (weights "q.norm", "k.norm" [head_dim]) and the turn
+    by position."""
+    hidden: int
+    n_heads: int
+    n_kv_heads: int
+    head_dim: int
+    v_dim: int
+    position: PositionSpec
+    scale: float
+    diff: float
+    conv: int
+    norm_eps: float
+    kind: str = "differential_attention"
+
+
+@dataclass(frozen=True)
+class FadingStateSpec:
+    """A matrix a head whose rows fade by a gate a channel and take in the gate's complement times v^T (HGRN2):
+    f = lower + (1 - lower) sigmoid(W_f h + b), S <- diag(f) S + (1 - f) v^T, o = S^T silu(W_q h), an RMS norm a head with
+    one weight of v_dim entries, W_o.  Tensors "q", "f", "f.b", "lower" [n_heads * head_dim], "v", "norm", "o"."""
+    hidden: int
+    n_heads: int
+    head_dim: int
+    v_dim: int
+    norm_eps: float
+    kind: str = "hgrn2"
+
+
+@dataclass(frozen=True)
 class GatedRecurrenceSpec:
     """The real-gated linear recurrent unit behind a causal convolution a channel, beside a GELU branch:
     y = gelu_tanh(W_y h + b), u = conv(W_x h + b); r, i = sigmoid of block-diagonal products of u (`blocks` equal
@@ -254,7 +289,8 @@ class RoutedExpertsSpec:
     choice only; the weights are the scores themselves.  `shared`: a `ClampedMlpSpec` that runs for every token beside
     the chosen experts (tensors under "shared."), its output added; `shared_gate`: times sigmoid(W_sg h), one number a
     token (tensor "shared.sg" [1, hidden], formed like a router's logit, in 32-bit).  `weight_on_input`: a chosen expert
-    runs on weight * h and its output is added as it is (instead of weight * expert(h))."""
+    runs on weight * h and its output is added as it is (instead of weight * expert(h)).  `activation` "silu": an expert is
+    W_down (silu(W_gate h) * (W_up h)), without limits."""
     hidden: int
     intermediate: int
     experts: int
@@ -270,6 +306,7 @@ class RoutedExpertsSpec:
     kind: str = "routed_experts"
     weight_on_input: bool = False
     shared_gate: bool = False
+    activation: str = "clamped"
 
 
 @dataclass(frozen=True)
@@ -313,6 +350,15 @@ class ParallelSpec:
 
 
 @dataclass(frozen=True)
+class GatedBranchSpec:
+    """How a layer's sub-layers stand around a stream kept in 32-bit that they read as it stands, each output gated and
+    normed before it enters: x <- x + norm(sub(x) * sigmoid(W x + b)), W and b stored under `gate_names` (one name a
+    sub-layer, mixer first) and that name + `bias_suffix`; `gate_names` None: no gates."""
+    gate_names: Optional[Tuple[str, ...]] = None
+    bias_suffix: str = ".b"
+
+
+@dataclass(frozen=True)
 class StreamsSpec:
     """How a layer's sub-layers stand around `streams` residual streams (kept in 32-bit): sub-layer q reads
     sum_s in_q[s] x_s through its norm, its output is scaled feature by feature (`layer_scale`), and the streams
@@ -338,7 +384,8 @@ class LayerSpec:
     layer without a feed-forward (`ffn` None, one norm); "post_norm" norms the stream after every sum (`residual`: a
     `PostNormSpec`; norms in the order behind the mixer, behind the feed-forward; one norm for a layer without one);
     "parallel" has ONE norm, whose output both sub-layers read, and adds their outputs together (`residual`: a
-    `ParallelSpec`).  `norms[i]` loads its weight from `norm_names[i]` (a norm with more tensors finds the others under
+    `ParallelSpec`); "gated_branch" norms what a sub-layer gives, behind an optional gate (`residual`: a `GatedBranchSpec`;
+    norms in the order of the sub-layers).  `norms[i]` loads its weight from `norm_names[i]` (a norm with more tensors finds the others under
     that name plus a suffix of its spec's)."""
     mixer: Any
     ffn: Any

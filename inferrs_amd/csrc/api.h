@@ -202,8 +202,8 @@ int ia_route_plan(int* order, int* tile_expert, int* tile_first, int* tile_rows,
                   int pairs, int E, int tile, hipStream_t stream);
 int ia_experts_gate_up(void* act, const void* h, const void* w_gu, const int* order, const int* tile_expert,
                        const int* tile_first, const int* tile_rows, const int* meta, int pairs, int E, int top,
-                       int W, int ff, float limit, float alpha, int tile, int tiled, const float* in_weight, int dtype,
-                       hipStream_t stream);
+                       int W, int ff, float limit, float alpha, int form, int tile, int tiled, const float* in_weight,
+                       int dtype, hipStream_t stream);
 int ia_experts_down(float* y, const void* act, const void* w_down, const int* order, const int* tile_expert,
                     const int* tile_first, const int* tile_rows, const int* meta, int pairs, int E, int W,
                     int ff, int tile, int tiled, int dtype, hipStream_t stream);
@@ -275,8 +275,35 @@ long long ia_linear_scan_workspace(int n_seqs, int max_q_len, int chunk, int H, 
 void ia_linear_scan_tune(int carry_mfma);
 // [o / (max(|den|, floor) + 1e-6)] [* act(gate)] -> RMS norm in groups of `group` features [* w] [* act(gate)]; act: 1 SiLU, 4 sigmoid
 int ia_group_norm_gate(void* out, const float* o, const float* den, const float* floor_, int head,
-                       const void* gate, long long g_ld, int g_off, int act, int gate_first, const float* w,
-                       float eps, int n, int inner, int group, int dtype, hipStream_t stream);
+                       const void* gate, long long g_ld, int g_off, int act, int gate_first, const float* w, int w_count,
+                       float eps, int n, int inner, int group, int dtype, hipStream_t stream);   // w: w_count entries, inner or group
+
+// A 32-bit residual stream that sub-layers read as it stands (gated_branch.hip): s = y1 + sum_k routed_w[k] routed[k] + y3_scale
+// y3; s *= sigmoid(gate + gate_b); x += s / sqrt(mean(s^2) + eps) * norm_w; xr (null: not wanted): the new x in g_dtype.
+// Every addend and the gate may be null.  y_dtype: of y1 and y3 (1 split, or 32-bit products still split along their k).
+int ia_branch_step(float* x, const void* y1, const void* y3, int y1_splits, int y3_splits, const float* y3_scale,
+                   const float* routed, const float* routed_w, int top, const void* gate, long long g_ld, int g_off,
+                   const float* gate_b, const float* norm_w, float eps, void* xr, int n, int W, int y_dtype,
+                   int g_dtype, hipStream_t stream);
+// Attention with several maps a head over shared values (map_attention.hip).  conv_qkv: rows [q | k | v | ...] through a
+// causal convolution a channel, per-map norm and turn of q and k, the cache writes; queries leave as [n, H maps, maps d],
+// zero outside their own map.  differ_norm: (a1 - lambda a2) / rms * scale a head, a [n, H, 2, dv].
+int ia_conv_qkv(void* q_out, void* k_cache, void* v_cache, const void* proj, long long ld, const void* taps, int k,
+                float* state, long long row_floats, long long tail_off, const float* q_norm_w, const float* k_norm_w,
+                float eps, const float* cos_t, const float* sin_t, int rot, int interleaved, const int* slots,
+                const int* token_seq, const int* cu_tokens, const int* state_slots, int n, int n_seqs, int H, int G,
+                int maps, int d, int dv, int page_size, int max_q_len, int dtype, hipStream_t stream);
+int ia_differ_norm(void* out, const void* a, float lambda, float eps, float scale, int n, int H, int dv, int dtype,
+                   hipStream_t stream);
+// S <- diag(f) S + (1 - f) v^T with f = lower + (1 - lower) sigmoid(z + f_bias) a channel, o = S^T silu(u) (fading_state.hip).
+// chunks 0: token by token, out 32-bit [n][H vdim] as it is; chunks > 0: 64 tokens side by side, that many chunks of a request
+// a pass, out normed a head (norm_w [vdim]) in the precision of proj (workspace: ia_fading_scan_workspace floats).
+int ia_fading_scan(void* out, float* state, long long row_floats, long long s_off, const void* proj, long long ld, int q_off,
+                   int f_off, int v_off, const float* f_bias, const float* lower, const float* norm_w, float eps,
+                   const int* cu_tokens, const int* state_slots, int n_seqs, int H, int dim, int vdim, int max_q_len,
+                   int chunks, float* workspace, int dtype, hipStream_t stream);
+int ia_fading_scan_fits(int dim, int vdim);
+long long ia_fading_scan_workspace(int n_seqs, int chunks, int H, int dim, int vdim);
 
 // Built per head size (-DIA_HEAD_DIM) into a library of its own.
 int ia_attention_mfma_head_dim(void);

@@ -206,7 +206,16 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(int* __restrict__ orde
     }
 }
 
-// act[place][j] = g' * sigmoid(alpha g') * (u' + 1), g' = min(gate_j . x, limit), u' = clamp(up_j . x, -limit, limit);
+// An expert's activation over its two sums.  Clamped: g' * sigmoid(alpha g') * (u' + 1), g' = min(g, limit), u' = clamp(u,
+// -limit, limit); plain (IA_EXPERT_SILU): silu(g) * u.  The choice is the same for all lanes of a launch.
+enum { IA_EXPERT_CLAMPED = 0, IA_EXPERT_SILU = 1 };
+__device__ __forceinline__ float expert_act(float g, float u, float limit, float alpha, int form) {
+    if (form == IA_EXPERT_SILU) return g / (1.0f + expf(-g)) * u;
+    const float gv = fminf(g, limit), uv = fminf(fmaxf(u, -limit), limit);
+    return gv / (1.0f + expf(-alpha * gv)) * (uv + 1.0f);
+}
+
+// act[place][j] = expert_act(gate_j . x, up_j . x);
 // x = h[pair / top] (times in_weight[pair], where given: 32-bit, one a pair).  w_gu [E][2 ff][W]: an expert's gate rows, then its up rows.
 template <typename T>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(T* __restrict__ act, const T* __restrict__ h,
@@ -215,7 +224,8 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(T* __restrict__ ac
                                                               const int* __restrict__ tile_first,
                                                               const int* __restrict__ tile_rows,
                                                               const int* __restrict__ meta, int top, int W, int ff,
-                                                              float limit, float alpha, const float* __restrict__ in_weight) {
+                                                              float limit, float alpha, int form,
+                                                              const float* __restrict__ in_weight) {
     __shared__ TileShared sh;
     const int tile = blockIdx.y;
     if (tile >= meta[0]) return;
@@ -235,8 +245,7 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(T* __restrict__ ac
         for (int b = 0; b < 4; ++b) {
             const int j = col0 + 4 * tx + b;
             if (j >= ff) continue;
-            const float gv = fminf(g[a][b] * wi, limit), uv = fminf(fmaxf(u[a][b] * wi, -limit), limit);
-            st(act + (long long)(first + i) * ff + j, gv / (1.0f + expf(-alpha * gv)) * (uv + 1.0f));
+            st(act + (long long)(first + i) * ff + j, expert_act(g[a][b] * wi, u[a][b] * wi, limit, alpha, form));
         }
     }
 }
@@ -281,7 +290,8 @@ __global__ __launch_bounds__(256) void experts_gate_up_mfma_kernel(bf16_t* __res
                                                                    const int* __restrict__ tile_first,
                                                                    const int* __restrict__ tile_rows,
                                                                    const int* __restrict__ meta, int top, int W, int ff,
-                                                                   float limit, float alpha, const float* __restrict__ in_weight) {
+                                                                   float limit, float alpha, int form,
+                                                              const float* __restrict__ in_weight) {
     using Tile = TileMfma<RT, FT, 64, true>;
     __shared__ typename Tile::Shared sh;
     const int tile = blockIdx.y;
@@ -306,8 +316,7 @@ __global__ __launch_bounds__(256) void experts_gate_up_mfma_kernel(bf16_t* __res
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 if (i >= rows || j0 + q >= ff) continue;
-                const float gv = fminf(gs[q] * wi, limit), uv = fminf(fmaxf(us[q] * wi, -limit), limit);
-                st(act + (long long)(first + i) * ff + j0 + q, gv / (1.0f + expf(-alpha * gv)) * (uv + 1.0f));
+                st(act + (long long)(first + i) * ff + j0 + q, expert_act(gs[q] * wi, us[q] * wi, limit, alpha, form));
             }
         }
     }
@@ -384,9 +393,10 @@ extern "C" int ia_route_plan(int* order, int* tile_expert, int* tile_first, int*
 
 extern "C" int ia_experts_gate_up(void* act, const void* h, const void* w_gu, const int* order, const int* tile_expert,
                                   const int* tile_first, const int* tile_rows, const int* meta, int pairs, int E, int top,
-                                  int W, int ff, float limit, float alpha, int tile, int tiled, const float* in_weight, int dtype,
-                                  hipStream_t stream) {
-    IA_CHECK(pairs >= 0 && W > 0 && ff > 0 && top >= 1 && limit > 0.f && (tile == 32 || tile == 64 || tile == 128), "experts_gate_up: bad sizes");
+                                  int W, int ff, float limit, float alpha, int form, int tile, int tiled, const float* in_weight,
+                                  int dtype, hipStream_t stream) {
+    IA_CHECK(form == IA_EXPERT_CLAMPED || form == IA_EXPERT_SILU, "experts_gate_up: unknown activation %d", form);
+    IA_CHECK(pairs >= 0 && W > 0 && ff > 0 && top >= 1 && (limit > 0.f || form == IA_EXPERT_SILU) && (tile == 32 || tile == 64 || tile == 128), "experts_gate_up: bad sizes");
     if (pairs == 0) return 0;
     IA_CHECK(!tiled || (dtype == IA_BF16 && W % 8 == 0 && tile_mfma_aligned(h) && tile_mfma_aligned(w_gu)),
              "experts_gate_up: weights stored as tiles are the matrix cores' (bfloat16, widths in steps of 8)");
@@ -396,19 +406,19 @@ extern "C" int ia_experts_gate_up(void* act, const void* h, const void* w_gu, co
     IA_CHECK(grid.y <= 65535, "experts_gate_up: %u row tiles are more than a grid takes", grid.y);
     if (tiled && tile == 128)
         experts_gate_up_mfma_kernel<8, 2><<<grid, 256, 0, stream>>>((bf16_t*)act, (const bf16_t*)h, (const bf16_t*)w_gu, order,
-                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, in_weight);
+                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, form, in_weight);
     else if (tiled && tile == 64)
         experts_gate_up_mfma_kernel<4, 2><<<grid, 256, 0, stream>>>((bf16_t*)act, (const bf16_t*)h, (const bf16_t*)w_gu, order,
-                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, in_weight);
+                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, form, in_weight);
     else if (tiled)
         experts_gate_up_mfma_kernel<2, 1><<<grid, 256, 0, stream>>>((bf16_t*)act, (const bf16_t*)h, (const bf16_t*)w_gu, order,
-                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, in_weight);
+                                                                    tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, form, in_weight);
     else if (dtype == IA_F32)
         experts_gate_up_kernel<float><<<grid, 256, 0, stream>>>((float*)act, (const float*)h, (const float*)w_gu, order,
-                                                                tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, in_weight);
+                                                                tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, form, in_weight);
     else
         experts_gate_up_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)act, (const bf16_t*)h, (const bf16_t*)w_gu, order,
-                                                                 tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, in_weight);
+                                                                 tile_expert, tile_first, tile_rows, meta, top, W, ff, limit, alpha, form, in_weight);
     IA_LAUNCH_CHECK("experts_gate_up");
     return 0;
 }

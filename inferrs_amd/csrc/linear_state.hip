@@ -901,7 +901,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void group_norm_gate_kernel(
     T* __restrict__ out, const float* __restrict__ o, const float* __restrict__ den, const float* __restrict__ floor_,
     int head, const T* __restrict__ gate, long long g_ld, int g_off, int act, int gate_first,
-    const float* __restrict__ w, float eps, int inner, int group, long long units) {
+    const float* __restrict__ w, int w_from, float eps, int inner, int group, long long units) {
     const long long unit = (long long)blockIdx.x * (blockDim.x / IA_WAVE) + threadIdx.x / IA_WAVE;
     if (unit >= units) return;
     const int lane = threadIdx.x & (IA_WAVE - 1);
@@ -926,7 +926,7 @@ __global__ __launch_bounds__(256) void group_norm_gate_kernel(
     const float rs = 1.0f / sqrtf(wave_sum(sq) / (float)group + eps);
     for (int c = c0 + lane; c < c0 + group; c += IA_WAVE) {
         float y = value(c) * rs;
-        if (w != nullptr) y *= w[c];
+        if (w != nullptr) y *= w[w_from ? c - c0 : c];
         if (gate != nullptr && !gate_first) y *= ls_gate(ld(gate + t * g_ld + g_off + c), act);
         st(out + t * inner + c, y);
     }
@@ -937,7 +937,7 @@ template <typename T>
 __global__ __launch_bounds__(1024) void group_norm_gate_block_kernel(
     T* __restrict__ out, const float* __restrict__ o, const float* __restrict__ den, const float* __restrict__ floor_,
     int head, const T* __restrict__ gate, long long g_ld, int g_off, int act, int gate_first,
-    const float* __restrict__ w, float eps, int inner, int group) {
+    const float* __restrict__ w, int w_from, float eps, int inner, int group) {
     __shared__ float scratch[16];
     const int per_row = inner / group;
     const long long t = blockIdx.x / per_row;
@@ -960,7 +960,7 @@ __global__ __launch_bounds__(1024) void group_norm_gate_block_kernel(
     const float rs = 1.0f / sqrtf(block_sum(sq, scratch) / (float)group + eps);
     for (int c = c0 + threadIdx.x; c < c0 + group; c += blockDim.x) {
         float y = value(c) * rs;
-        if (w != nullptr) y *= w[c];
+        if (w != nullptr) y *= w[w_from ? c - c0 : c];
         if (gate != nullptr && !gate_first) y *= ls_gate(ld(gate + t * g_ld + g_off + c), act);
         st(out + t * inner + c, y);
     }
@@ -968,9 +968,12 @@ __global__ __launch_bounds__(1024) void group_norm_gate_block_kernel(
 
 extern "C" int ia_group_norm_gate(void* out, const float* o, const float* den, const float* floor_, int head,
                                   const void* gate, long long g_ld, int g_off, int act, int gate_first, const float* w,
-                                  float eps, int n, int inner, int group, int dtype, hipStream_t stream) {
+                                  int w_count, float eps, int n, int inner, int group, int dtype, hipStream_t stream) {
     IA_CHECK(n >= 0 && inner > 0 && group > 0 && inner % group == 0 && head > 0 && inner % head == 0,
              "group_norm_gate: %d features in groups of %d, heads of %d", inner, group, head);
+    IA_CHECK(w == nullptr || w_count == inner || w_count == group, "group_norm_gate: a weight of %d entries for %d features in groups of %d",
+             w_count, inner, group);
+    const int w_from = w_count == group ? 1 : 0;               // (one weight for every group alike)
     IA_CHECK((den == nullptr) == (floor_ == nullptr), "group_norm_gate: a normaliser and its floor come together");
     IA_CHECK(gate == nullptr || ((act == IA_ACT_SILU || act == 4) && g_off >= 0 && g_off + inner <= g_ld),
              "group_norm_gate: gate activation %d (1 SiLU, 4 sigmoid) at %d of %lld", act, g_off, g_ld);
@@ -983,21 +986,21 @@ extern "C" int ia_group_norm_gate(void* out, const float* o, const float* den, c
         const int threads = group >= 4096 ? 1024 : group >= 2048 ? 512 : 256;
         if (dtype == IA_F32)
             group_norm_gate_block_kernel<float><<<(unsigned)units, threads, 0, stream>>>((float*)out, o, den, floor_, head, (const float*)gate,
-                                                                                  g_ld, g_off, act, gate_first, w, eps, inner, group);
+                                                                                  g_ld, g_off, act, gate_first, w, w_from, eps, inner, group);
         else
             group_norm_gate_block_kernel<bf16_t><<<(unsigned)units, threads, 0, stream>>>((bf16_t*)out, o, den, floor_, head,
                                                                                    (const bf16_t*)gate, g_ld, g_off, act, gate_first, w,
-                                                                                   eps, inner, group);
+                                                                                   w_from, eps, inner, group);
         IA_LAUNCH_CHECK("group_norm_gate (blocks)");
         return 0;
     }
     const unsigned blocks = (unsigned)((units + 3) / 4);
     if (dtype == IA_F32)
         group_norm_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)out, o, den, floor_, head, (const float*)gate, g_ld, g_off,
-                                                                  act, gate_first, w, eps, inner, group, units);
+                                                                  act, gate_first, w, w_from, eps, inner, group, units);
     else
         group_norm_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)out, o, den, floor_, head, (const bf16_t*)gate, g_ld,
-                                                                   g_off, act, gate_first, w, eps, inner, group, units);
+                                                                   g_off, act, gate_first, w, w_from, eps, inner, group, units);
     IA_LAUNCH_CHECK("group_norm_gate");
     return 0;
 }

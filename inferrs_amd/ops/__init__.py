@@ -1253,3 +1253,5 @@ from .mix import (clamped_gate_mul, conv_step, embed_gather_scaled, experts_forw
 from .state import (activation, conv_act_step, exp_gates, group_norm_gate, linear_scan, sandwich_step,   # noqa: E402
                     step_gates)
 from . import state                                                                                    # noqa: E402
+from .gated import branch_step, conv_qkv, differ_norm, fading_scan                                     # noqa: E402
+from . import gated                                                                                    # noqa: E402

@@ -18,6 +18,7 @@ ROW_TILE = 32                 # rows of a tile of the grouped products
 LARGE_TILE = int(os.environ.get("INFERRS_AMD_EXPERT_TILE", "64"))     # rows of the matrix cores' large tile: 64 or 128
 LARGE_TILE_FROM = 0.75        # rows an expert (on average), in large tiles, from which the experts' products take them
 SCORE_FUNCTIONS = {"sigmoid": 0, "softmax": 1}
+EXPERT_ACTIVATIONS = {"clamped": 0, "silu": 1}
 
 
 # ---- residual streams -----------------------------------------------------------------------
@@ -265,11 +266,12 @@ def experts_tiled_fits(dtype: torch.dtype, width: int, ff: int) -> bool:
 
 
 def experts_forward(h: torch.Tensor, sel: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-                    limit: float, alpha: float, ff: Optional[int] = None, in_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    limit: float, alpha: float, ff: Optional[int] = None, in_weight: Optional[torch.Tensor] = None,
+                    activation: str = "clamped") -> torch.Tensor:
     """The chosen experts of every row: w_gate_up [E, 2 ff, width] (gate rows, then up rows), w_down [E, width, ff],
     or both as tiles (`tile_weights` of [E, 2, ff, width] and of [E, width, ff]; then `ff` is given);
-    act = g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit).  Returns one
-    32-bit output row a (row, k) pair, [n, top, width]; nothing is added up here.  A choice of E or beyond names no
+    act = g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit); with `activation`
+    "silu" silu(g) * u, without limits.  Returns one 32-bit output row a (row, k) pair, [n, top, width]; nothing is added up here.  A choice of E or beyond names no
     expert with weights: its row is left unwritten (whoever adds the rows up knows what stands for it).  `in_weight`
     [n, top] (32-bit): pair (row, k) runs its expert on in_weight[row, k] * h[row] (the factor meets the two products'
     32-bit sums ahead of the limits, which is the same number)."""
@@ -305,7 +307,7 @@ def experts_forward(h: torch.Tensor, sel: torch.Tensor, w_gate_up: torch.Tensor,
     _check(lib.ia_route_plan(_p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta), _p(sel), pairs, E, tile, _stream()))
     act = torch.empty((pairs, ff), dtype=h.dtype, device=h.device)
     _check(lib.ia_experts_gate_up(_p(act), _p(h), _p(w_gate_up), _p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta),
-                                  pairs, E, top, W, ff, ctypes.c_float(limit), ctypes.c_float(alpha), tile, int(tiled),
+                                  pairs, E, top, W, ff, ctypes.c_float(limit), ctypes.c_float(alpha), EXPERT_ACTIVATIONS[activation], tile, int(tiled),
                                   _p(in_weight), _dt(h), _stream()))
     y = torch.empty((n, top, W), dtype=torch.float32, device=h.device)
     _check(lib.ia_experts_down(_p(y), _p(act), _p(w_down), _p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta), pairs,

@@ -191,11 +191,12 @@ def group_norm_gate(o: torch.Tensor, *, group: int, head: int, eps: float, out_d
                     floor: Optional[torch.Tensor] = None) -> torch.Tensor:
     """What follows a recurrence: o [n, inner] (32-bit) is divided by max(|den|, floor) + 1e-6 a (token, head of `head`
     features) when `den` is given, multiplied by act(gate[:, gate_off ...]) before (`gate_first`) or behind an RMS norm over
-    groups of `group` neighbouring features with `weight`; returns [n, inner] in `out_dtype`."""
+    groups of `group` neighbouring features with `weight` [inner], or [group] for every group alike; returns [n, inner] in
+    `out_dtype`."""
     _dev(o, weight, gate, den, floor)
     _f32(o, "o"); _f32(weight, "weight"); _f32(den, "den"); _f32(floor, "floor")
     n, inner = o.shape
-    if inner % group or inner % head or (weight is not None and weight.numel() != inner):
+    if inner % group or inner % head or (weight is not None and weight.numel() not in (inner, group)):
         raise KernelError(f"group_norm_gate: {inner} features in groups of {group}, heads of {head}")
     if gate is not None and (gate.dim() != 2 or gate.shape[0] != n or gate.dtype != out_dtype):
         raise KernelError("group_norm_gate: the gate is 2-D rows in the precision of the result")
@@ -204,7 +205,8 @@ def group_norm_gate(o: torch.Tensor, *, group: int, head: int, eps: float, out_d
     out = torch.empty((n, inner), dtype=out_dtype, device=o.device)
     _check(library().ia_group_norm_gate(
         _p(out), _p(o), _p(den), _p(floor), head, _p(gate), gate.shape[1] if gate is not None else 0, gate_off, act,
-        int(gate_first), _p(weight), ctypes.c_float(eps), n, inner, group, _DT[out_dtype], _stream()))
+        int(gate_first), _p(weight), weight.numel() if weight is not None else inner, ctypes.c_float(eps), n, inner, group,
+        _DT[out_dtype], _stream()))
     return out
 
 

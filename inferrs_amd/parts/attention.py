@@ -188,8 +188,11 @@ class Attention(Mixer):
         return self._project(ctx, joined)
 
     def _attend(self, ctx, q, cache, group):
+        return self.attend(self.spec, ctx, q, cache, group)
+
+    @staticmethod
+    def attend(s: AttentionSpec, ctx, q, cache, group):
         """The paged attention of the step's queries: the matrix cores where they take the sizes, else the plain kernel."""
-        s = self.spec
         if ops.attention_mfma_fits(q.dtype, s.head_dim, group.page_size, s.value_dim):
             common = dict(window=s.window, scale=s.softmax_scale, sink=s.sink, mask_chunk=s.mask_chunk)
             if 0 < ctx.n_single < ctx.n_seqs:

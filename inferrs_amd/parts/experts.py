@@ -13,7 +13,8 @@ the stream's own row takes their place); `correction`, a vector added to the sco
 feed-forward of the experts' form that runs for every token (`ClampedMlp`; its output rides along as `RoutedRows.extra`),
 behind a sigmoid gate a token with `shared_gate` (its row stands behind the router's in one matrix, so that the gate is
 formed like a router's logit: `RoutedRows.extra_scale`); `weight_on_input`, a chosen expert runs on weight * h and its
-output counts as it is (`RoutedRows.weights` is None then)."""
+output counts as it is (`RoutedRows.weights` is None then); `activation` "silu", experts without limits,
+W_down (silu(W_gate h) * (W_up h))."""
 from __future__ import annotations
 
 from typing import Dict
@@ -77,6 +78,8 @@ class RoutedExperts(FeedForward):
                             f"input on (up to {ops.mix.MAX_TOP} of {ops.mix.MAX_EXPERTS})")
         if spec.score not in ops.mix.SCORE_FUNCTIONS:
             raise SpecError(f"routed_experts: score {spec.score!r} has no kernel (known: {sorted(ops.mix.SCORE_FUNCTIONS)})")
+        if spec.activation not in ops.mix.EXPERT_ACTIVATIONS:
+            raise SpecError(f"routed_experts: activation {spec.activation!r} has no kernel (known: {sorted(ops.mix.EXPERT_ACTIVATIONS)})")
         self.spec = spec
         # the router's logits are 32-bit sums whatever its matrix is stored in (`ops.route`)
         self.router = to_compute(tensors["router"], dtype, device)
@@ -116,7 +119,7 @@ class RoutedExperts(FeedForward):
             sel, weights = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction)
         rows = ops.experts_forward(h, sel, self.gate_up, self.down, s.limit, s.alpha,
                                    ff=s.intermediate if self.tiled else None,
-                                   in_weight=weights if s.weight_on_input else None)
+                                   in_weight=weights if s.weight_on_input else None, activation=s.activation)
         extra = self.shared.forward(ctx, h) if self.shared is not None else None
         if s.weight_on_input:
             weights = None

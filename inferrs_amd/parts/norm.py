@@ -22,14 +22,15 @@ class RMSNorm(Norm):
 
     @classmethod
     def tensors(cls, spec: NormSpec) -> Dict[str, TensorSpec]:
-        return {"weight": TensorSpec((spec.size,), "norm")}
+        return {"weight": TensorSpec(() if spec.scalar else (spec.size,), "norm")}
 
     def __init__(self, spec: NormSpec, tensors: Dict[str, torch.Tensor], dtype, device):
         self.spec = spec
         self.eps = float(spec.eps)
         self.add_one = bool(spec.add_one)
         # Norm weights are vectors: kept in 32-bit whatever the activations are stored in.
-        self.weight = tensors["weight"].to(device=device, dtype=torch.float32).contiguous()
+        weight = tensors["weight"].to(device=device, dtype=torch.float32)
+        self.weight = (weight.expand(spec.size) if spec.scalar else weight).contiguous()
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return ops.rmsnorm(x, self.weight, self.eps, self.add_one)
