@@ -74,7 +74,7 @@ class VufizenConfig:
         """For every layer of config.json the layer whose tensors it uses (itself unless it says `weights_of`)."""
         layers = self.raw["layers"]
         out: List[int] = []
-        for i, layer in enumerate(layers):
+        for i in range(len(layers)):
             j, seen = i, {i}
             while layers[j].get("weights_of") is not None:
                 where = f"layers[{j}]"
@@ -83,9 +83,6 @@ class VufizenConfig:
                     raise ConfigError(f"config.json: '{where}.weights_of' = {k} must lead to a layer with tensors of its own")
                 seen.add(k)
                 j = k
-            for key in ("type", "mixer", "mlp"):
-                if layer.get(key) != layers[j].get(key):
-                    raise ConfigError(f"config.json: 'layers[{i}].{key}' differs from layer {j}'s, whose tensors it uses")
             out.append(j)
         return out
 
@@ -165,6 +162,10 @@ class VufizenConfig:
             layers.append(LayerSpec(mixer=self._mixer(i, layer, hidden, eps), ffn=ffn, norms=(norm,) * len(branches),
                                     norm_names=tuple(p + "norm" + b for b in branches), mixer_prefix=p + "mix.", ffn_prefix=p + "mlp.",
                                     arrangement="gated_branch", residual=GatedBranchSpec(tuple(p + "rg" + b for b in branches))))
+        for i, j in enumerate(owners):
+            for key in ("type", "mixer", "mlp"):
+                if layers_raw[i].get(key) != layers_raw[j].get(key):
+                    raise ConfigError(f"config.json: 'layers[{i}].{key}' differs from layer {j}'s, whose tensors it uses")
         max_position = int(raw.get("max_position") or DEFAULT_MAX_POSITION)
         return ModelSpec(
             architecture=self.architecture, vocab_size=vocab, hidden=hidden, layers=tuple(layers),
