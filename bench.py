@@ -18,7 +18,7 @@ choice): `mixed16` is 16 requests with prompts of 128 to 4,096 random tokens in 
 `--decode-tokens` tokens.  Its JSON line gives tokens a second over the whole run, the prompts' and the
 decoded tokens' rates apart, and the time to a request's first token.
 
-    python bench.py --design buketar|lofudra|fisanex|ligizen [--design-shapes 1k,2k,4k]
+    python bench.py --design buketar|lofudra|fisanex|ligizen|vufizen [--design-shapes 1k,2k,4k]
 
 measures the Buketar design (latent attention, gated recurrences, routed experts, residual streams), the Lofudra
 design (windowed sink attention beside retention, matrix memory, state space, norms on both sides) or the Fisanex design
@@ -26,7 +26,9 @@ design (windowed sink attention beside retention, matrix memory, state space, no
 routed experts with outputs that hand the input on and a shared expert) at a few layer
 sizes beside the dense decoder at equal width, layers and feed-forward products a token, or the Ligizen design (one layer
 norm a layer that both sub-layers read, latent window attention with learned sinks beside chunked attention over caches
-that layers share, experts weighted on their inputs, a token's own input a layer) beside the Fisanex design at equal size: prompts of `--prefill-tokens`
+that layers share, experts weighted on their inputs, a token's own input a layer) beside the Fisanex design at equal size,
+or the Vufizen design (gated, normed branches; differential attention behind a short convolution beside a matrix state that fades
+by a gate a channel; routed experts in every layer) beside the Fisanex and the Lofudra design at equal width and layers: prompts of `--prefill-tokens`
 tokens, decode steps at `--batch` and at batch 1 through the serving loop, and every kernel's time in one prompt and one
 decode step of both.  One JSON line; the default record above is not touched by it.
 
@@ -500,9 +502,35 @@ LIGIZEN_LIKE_KERNEL = {"parallel_step": "postnorm_step", "qk_rope_kv_strided": "
                        "softcap": "scale", "embed_gather": "embed_gather_scaled"}
 
 
+# ---- the Vufizen design beside the Fisanex and the Lofudra design at equal size (`--design vufizen`) -------------
+# Layer sizes in the range of real models of its kind.  Even layers: differential attention with maps of 64 (keys of 128 a
+# head), values of 128 and a quarter as many key heads, a convolution of four taps; odd layers: the fading matrix state in
+# heads of 128 x 128; every layer routed experts (32, 4 a token) with a shared expert of twice their size behind its gate.
+# The twins are the package's closest relatives: the Fisanex design (grouped attention with keys of 128, the same experts in
+# every other layer) and the Lofudra design (recurrences with a matrix state a head in every layer).
+def vufizen_shape(width: int, layers: int, vocab: int = 32768):
+    heads, ff = width // 128, 3 * width // 4 // 64 * 64
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 128, "scale": 0.125,
+                                          "conv": 4, "diff": 0.5, "rot": {"base": 500000.0, "dims": 64}}}
+    rec = {"type": "hgrn2", "mixer": {"heads": heads, "dim": 128, "vdim": 128}}
+    mlp = {"kind": "moe", "router": {"experts": 32, "top": 4}, "expert": {"ff": ff}, "shared": {"ff": 2 * ff}}
+    return {"architecture": "Vufizen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "layers": [dict(att if i % 2 == 0 else rec, mlp=mlp) for i in range(layers)]}
+
+
+def vufizen_twins(b: dict, vocab: int = 32768) -> dict:
+    return {"fisanex": fisanex_shape(b["width"], b["layers"], vocab), "lofudra": lofudra_shape(b["width"], b["layers"], vocab)}
+
+
+VUFIZEN_LIKE_KERNEL = {"branch_step": "postnorm_step", "conv_qkv": "qk_rope_kv_strided", "differ_norm": "sigmoid_gate",
+                       "fading_scan": "linear_scan", "group_norm_gate": "group_norm_gate", "experts_gate_up": "experts_gate_up",
+                       "experts_down": "experts_down", "route": "route", "route_plan": "route_plan",
+                       "attention_mfma": "attention_mfma", "gate_mul": "clamped_gate_mul", "parallel_step": "postnorm_step"}
+
+
 def design_main(args) -> int:
-    """Prefill and decode throughput of a design at a few layer sizes beside the dense decoder at equal
-    size (random weights), and the time of every kernel of one prefill and one decode step of both."""
+    """Prefill and decode throughput of a design at a few layer sizes beside the dense decoder (or the designs that
+    are closer to it) at equal size (random weights), and the time of every kernel of one prefill and one decode step of each."""
     import torch
     from inferrs_amd.config import Qwen3Config
     from inferrs_amd.config.buketar import BuketarConfig
@@ -512,7 +540,13 @@ def design_main(args) -> int:
     batch, context, prompt = args.batch, min(args.context, 2048), args.prefill_tokens
     records = {}
     twin_label, twin_cls, twin_vocab = "dense", Qwen3Config, "vocab_size"
-    if args.design == "ligizen":
+    twins_of = None                              # raw -> {label: raw} where a design stands beside several others
+    if args.design == "vufizen":
+        from inferrs_amd.config.vufizen import VufizenConfig
+        shapes, shape_of, config_cls, like = FISANEX_SHAPES, vufizen_shape, VufizenConfig, VUFIZEN_LIKE_KERNEL
+        title, beside = "Vufizen", "Fisanex and Lofudra at equal width and layers"
+        twins_of, twin_classes = vufizen_twins, {"fisanex": FisanexConfig, "lofudra": LofudraConfig}
+    elif args.design == "ligizen":
         from inferrs_amd.config.ligizen import LigizenConfig
         shapes, shape_of, twin_of, config_cls, like = FISANEX_SHAPES, ligizen_shape, ligizen_twin, LigizenConfig, LIGIZEN_LIKE_KERNEL
         title, beside = "Ligizen", "Fisanex at equal width and layers"
@@ -528,10 +562,14 @@ def design_main(args) -> int:
         title, beside = "Buketar", "Qwen3 dense at equal width, layers and feed-forward products a token"
     for name in (args.design_shapes.split(",") if args.design_shapes else sorted(shapes)):
         b = shapes[name]
-        raw_new, raw_old = shape_of(**b), twin_of(b)
+        raw_new = shape_of(**b)
+        if twins_of is not None:
+            beside_it = [(label, twin_classes[label].from_dict(raw), raw["vocab"]) for label, raw in twins_of(b).items()]
+        else:
+            raw_old = twin_of(b)
+            beside_it = [(twin_label, twin_cls.from_dict(raw_old), raw_old[twin_vocab])]
         rec = {}
-        for label, config, vocab in ((args.design, config_cls.from_dict(raw_new), raw_new["vocab"]),
-                                     (twin_label, twin_cls.from_dict(raw_old), raw_old[twin_vocab])):
+        for label, config, vocab in [(args.design, config_cls.from_dict(raw_new), raw_new["vocab"])] + beside_it:
             pages = batch * (-(-context // PAGE) + 1) + -(-prompt // PAGE) + 8
             note(f"{name} {label}: random weights, {pages} pages")
             engine = Engine.from_random(config, seed=0, dtype=args.dtype, page_size=PAGE, num_pages=pages, max_seqs=batch + 1)
@@ -587,9 +625,10 @@ def main() -> int:
                     help="workloads: cut prompt portions so that a step's tokens are a multiple of this (0: off)")
     ap.add_argument("--decode-run", type=int, default=8,
                     help="decode steps that the serving loop queues on the GPU at once (1: one at a time)")
-    ap.add_argument("--design", default=None, choices=["buketar", "lofudra", "fisanex", "ligizen"],
+    ap.add_argument("--design", default=None, choices=["buketar", "lofudra", "fisanex", "ligizen", "vufizen"],
                     help="instead of the headline: prefill and decode throughput of this design at a few layer sizes "
-                         "beside the dense decoder (ligizen: beside the Fisanex design) at equal size, with every kernel's time")
+                         "beside the dense decoder (ligizen: beside the Fisanex design; vufizen: beside the Fisanex and the Lofudra design) "
+                         "at equal size, with every kernel's time")
     ap.add_argument("--design-shapes", default=None, help="with --design: the sizes to run, with commas (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:

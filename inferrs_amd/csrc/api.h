@@ -302,7 +302,6 @@ int ia_fading_scan(void* out, float* state, long long row_floats, long long s_of
                    int f_off, int v_off, const float* f_bias, const float* lower, const float* norm_w, float eps,
                    const int* cu_tokens, const int* state_slots, int n_seqs, int H, int dim, int vdim, int max_q_len,
                    int chunks, float* workspace, int dtype, hipStream_t stream);
-int ia_fading_scan_fits(int dim, int vdim);
 long long ia_fading_scan_workspace(int n_seqs, int chunks, int H, int dim, int vdim);
 
 // Built per head size (-DIA_HEAD_DIM) into a library of its own.

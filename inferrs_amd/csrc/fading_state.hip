@@ -476,8 +476,6 @@ __global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const Fad
         }
 }
 
-extern "C" int ia_fading_scan_fits(int dim, int vdim) { return dim <= FS_MAX_DIM && vdim <= FS_MAX_VDIM ? 1 : 0; }
-
 // Floats of workspace for passes of `chunks` chunks a request.
 extern "C" long long ia_fading_scan_workspace(int n_seqs, int chunks, int H, int dim, int vdim) {
     return (long long)n_seqs * chunks * ((long long)H * vdim * dim + (long long)H * dim);
@@ -544,7 +542,7 @@ extern "C" int ia_fading_scan(void* out, float* state, long long row_floats, lon
         IA_LAUNCH_CHECK("fading_scan");
         return 0;
     }
-    IA_CHECK(ia_fading_scan_fits(dim, vdim) && workspace != nullptr && norm_w != nullptr && chunks > 0,
+    IA_CHECK(dim <= FS_MAX_DIM && vdim <= FS_MAX_VDIM && workspace != nullptr && norm_w != nullptr && chunks > 0,
              "fading_scan: chunks take keys up to %d, values up to %d, a workspace and the norm's weight", FS_MAX_DIM, FS_MAX_VDIM);
     IA_CHECK((long long)n_seqs * chunks <= 65535 && H <= 65535, "fading_scan: %d requests x %d chunks exceed the grid", n_seqs, chunks);
     const int d16 = (dim + 15) / 16 * 16, ld_s = d16 + 4;

@@ -13,6 +13,7 @@ from . import KernelError, _DT, _check, _check_cache, _dev, _dt, _f32, _i32, _p,
 from .mix import MAX_TOP
 
 FADING_MAX_DIM = 512              # rows of a head's matrix that the walk takes
+FADING_CHUNK_DIM, FADING_CHUNK_VDIM = 128, 256      # keys and values that the chunks take
 FADING_CHUNK = 64                 # tokens of a chunk when long portions run in chunks side by side
 FADING_CHUNKS_FROM = 128          # steps whose longest portion has more tokens than this run in chunks
 FADING_WORKSPACE_FLOATS = 1 << 28     # a pass over the chunks takes no more than this (1 GiB): more passes beyond
@@ -152,7 +153,7 @@ def fading_scan(proj: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads
         raise KernelError(f"fading_scan: a key size of {dim} is beyond {FADING_MAX_DIM}")
     lib = library()
     n_seqs, longest = state_slots.numel(), int(max_q_len) or n
-    fits = bool(lib.ia_fading_scan_fits(dim, vdim))
+    fits = dim <= FADING_CHUNK_DIM and vdim <= FADING_CHUNK_VDIM
     if chunks is None:
         chunks = fits and longest > FADING_CHUNKS_FROM
     elif chunks and not fits:
