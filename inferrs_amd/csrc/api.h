@@ -195,8 +195,14 @@ int ia_rglru_scan_chunked(void* out, float* state, float* work, const float* u, 
 // choice_bias: null, or [E] 32-bit values that count in the choice only (score + bias picks, the score weighs).  The plan
 // gives a pair whose choice is E or beyond (an output of the router that names no expert with weights) no place and no tile.
 int ia_route(int* sel, float* weight, const void* h, const void* router, int n, int W, int E, int top,
-             float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int dtype,
-             hipStream_t stream);
+             float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order,
+             int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, int dtype, hipStream_t stream);   // order: null, or the plan of ia_route_plan as well
+// the choice from logits that a product has left (32-bit rows of pitch ld from column off on: E experts, then the gates), up to
+// 16 tokens in one block, with the plan
+int ia_route_logits(int* sel, float* weight, const float* logits, long long ld, int off, int n, int E, int top, float scale,
+                    int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order, int* tile_expert,
+                    int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, hipStream_t stream);
+int ia_route_plans(int n, int W, int rows, int dtype, const void* h, const void* router);    // 1: ia_route makes this step's plan itself
 int ia_route_tiles(int pairs, int E);
 int ia_route_plan(int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, const int* sel,
                   int pairs, int E, int tile, hipStream_t stream);
@@ -279,12 +285,12 @@ int ia_group_norm_gate(void* out, const float* o, const float* den, const float*
                        float eps, int n, int inner, int group, int dtype, hipStream_t stream);   // w: w_count entries, inner or group
 
 // A 32-bit residual stream that sub-layers read as it stands (gated_branch.hip): s = y1 + sum_k routed_w[k] routed[k] + y3_scale
-// y3; s *= sigmoid(gate + gate_b); x += s / sqrt(mean(s^2) + eps) * norm_w; xr (null: not wanted): the new x in g_dtype.
+// y3; s *= sigmoid(gate + gate_b); x += s / sqrt(mean(s^2) + eps) * norm_w; xr (null: not wanted): the new x in x_dtype.
 // Every addend and the gate may be null.  y_dtype: of y1 and y3 (1 split, or 32-bit products still split along their k).
 int ia_branch_step(float* x, const void* y1, const void* y3, int y1_splits, int y3_splits, const float* y3_scale,
                    const float* routed, const float* routed_w, int top, const void* gate, long long g_ld, int g_off,
                    const float* gate_b, const float* norm_w, float eps, void* xr, int n, int W, int y_dtype,
-                   int g_dtype, hipStream_t stream);
+                   int g_dtype, int x_dtype, hipStream_t stream);
 // Attention with several maps a head over shared values (map_attention.hip).  conv_qkv: rows [q | k | v | ...] through a
 // causal convolution a channel, per-map norm and turn of q and k, the cache writes; queries leave as [n, H maps, maps d],
 // zero outside their own map.  differ_norm: (a1 - lambda a2) / rms * scale a head, a [n, H, 2, dv].

@@ -34,6 +34,90 @@ __device__ __forceinline__ void load8(const bf16_t* p, float (&v)[8]) {
     }
 }
 
+// One wave: a token's choice and weights from its logits (of E rows of the router's matrix, the last `gates` of which take no
+// part in it).  Q: registers of logits a lane (E - gates up to 64 Q).
+template <int Q>
+__device__ __forceinline__ void route_pick(int* __restrict__ sel, float* __restrict__ weight, const float* logits, int t, int lane, int E,
+                                           int top, float scale, int score_fn, int renorm, const float* __restrict__ choice_bias,
+                                           int gates, float* __restrict__ gate_out, int* chosen = nullptr) {
+    if (gates > 0) {
+        E -= gates;
+        for (int j = lane; j < gates; j += IA_WAVE) gate_out[(long long)t * gates + j] = 1.0f / (1.0f + expf(-logits[E + j]));
+    }
+    float z[Q];             // expert e lives in lane e % 64, register e / 64
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int e = q * IA_WAVE + lane;
+        z[q] = e < E ? logits[e] : -INFINITY;
+    }
+    float zmax = -INFINITY, denom = 1.f;
+    if (score_fn == IA_SCORE_SOFTMAX) {
+#pragma unroll
+        for (int q = 0; q < Q; ++q) zmax = fmaxf(zmax, z[q]);
+        zmax = wave_max(zmax);
+        float s = 0.f;
+#pragma unroll
+        for (int q = 0; q < Q; ++q) s += z[q] > -INFINITY ? expf(z[q] - zmax) : 0.f;
+        denom = wave_sum(s);
+    }
+    float total = 0.f, mine = 0.f;
+    int mine_e = 0;
+    if (choice_bias != nullptr) {
+        // The choice goes by score + bias, the weights by the score alone: the scores are formed first, and the picking
+        // walks the biased ones (of equal ones the lower index).
+        float sc[Q], key[Q];
+#pragma unroll
+        for (int q = 0; q < Q; ++q) {
+            const int e = q * IA_WAVE + lane;
+            sc[q] = e < E ? (score_fn == IA_SCORE_SOFTMAX ? expf(z[q] - zmax) / denom : 1.0f / (1.0f + expf(-z[q]))) : 0.f;
+            key[q] = e < E ? sc[q] + choice_bias[e] : -INFINITY;
+        }
+        for (int k = 0; k < top; ++k) {
+            float best = -INFINITY, best_s = 0.f;
+            int best_e = 0x7fffffff;
+#pragma unroll
+            for (int q = 0; q < Q; ++q)
+                if (key[q] > best) { best = key[q]; best_e = q * IA_WAVE + lane; best_s = sc[q]; }
+#pragma unroll
+            for (int o = IA_WAVE / 2; o > 0; o >>= 1) {
+                const float ob = __shfl_xor(best, o, IA_WAVE), os = __shfl_xor(best_s, o, IA_WAVE);
+                const int oe = __shfl_xor(best_e, o, IA_WAVE);
+                if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; best_s = os; }
+            }
+#pragma unroll
+            for (int q = 0; q < Q; ++q)
+                if (best_e == q * IA_WAVE + lane) key[q] = -INFINITY;
+            total += best_s;
+            if (lane == k) { mine = best_s; mine_e = best_e; }
+        }
+    } else
+    for (int k = 0; k < top; ++k) {
+        // every lane's best, then the wave's: the largest logit, of equal ones the lower index
+        float best = -INFINITY;
+        int best_e = 0x7fffffff;
+#pragma unroll
+        for (int q = 0; q < Q; ++q)
+            if (z[q] > best) { best = z[q]; best_e = q * IA_WAVE + lane; }
+#pragma unroll
+        for (int o = IA_WAVE / 2; o > 0; o >>= 1) {
+            const float ob = __shfl_xor(best, o, IA_WAVE);
+            const int oe = __shfl_xor(best_e, o, IA_WAVE);
+            if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; }
+        }
+#pragma unroll
+        for (int q = 0; q < Q; ++q)
+            if (best_e == q * IA_WAVE + lane) z[q] = -INFINITY;
+        const float s = score_fn == IA_SCORE_SOFTMAX ? expf(best - zmax) / denom : 1.0f / (1.0f + expf(-best));
+        total += s;
+        if (lane == k) { mine = s; mine_e = best_e; }
+    }
+    if (lane < top) {
+        sel[(long long)t * top + lane] = mine_e;
+        if (chosen != nullptr) chosen[lane] = mine_e;
+        weight[(long long)t * top + lane] = (renorm ? mine / total : mine) * scale;
+    }
+}
+
 #define IA_ROUTE_WAVES 4        // waves of a token's block
 #define IA_ROUTE_FEW_TOKENS 64 // up to this many tokens a step the blocks are too few to hide a wave's chain of loads
 #define IA_ROUTE_SHARE 8        // experts whose sums a wave holds at a time: a block takes 32 experts a round (routers of 33 to 64
@@ -92,88 +176,18 @@ __global__ __launch_bounds__(64 * WAVES) void route_kernel(int* __restrict__ sel
     }
     __syncthreads();
     if (wave != 0) return;
-    if (gates > 0) {
-        E -= gates;
-        for (int j = lane; j < gates; j += IA_WAVE) gate_out[(long long)t * gates + j] = 1.0f / (1.0f + expf(-logits[E + j]));
-    }
-    float z[IA_MAX_EXPERTS / IA_WAVE];             // expert e lives in lane e % 64, register e / 64
-#pragma unroll
-    for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q) {
-        const int e = q * IA_WAVE + lane;
-        z[q] = e < E ? logits[e] : -INFINITY;
-    }
-    float zmax = -INFINITY, denom = 1.f;
-    if (score_fn == IA_SCORE_SOFTMAX) {
-#pragma unroll
-        for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q) zmax = fmaxf(zmax, z[q]);
-        zmax = wave_max(zmax);
-        float s = 0.f;
-#pragma unroll
-        for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q) s += z[q] > -INFINITY ? expf(z[q] - zmax) : 0.f;
-        denom = wave_sum(s);
-    }
-    float total = 0.f, mine = 0.f;
-    int mine_e = 0;
-    if (choice_bias != nullptr) {
-        // The choice goes by score + bias, the weights by the score alone: the scores are formed first, and the picking
-        // walks the biased ones (of equal ones the lower index).
-        float sc[IA_MAX_EXPERTS / IA_WAVE], key[IA_MAX_EXPERTS / IA_WAVE];
-#pragma unroll
-        for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q) {
-            const int e = q * IA_WAVE + lane;
-            sc[q] = e < E ? (score_fn == IA_SCORE_SOFTMAX ? expf(z[q] - zmax) / denom : 1.0f / (1.0f + expf(-z[q]))) : 0.f;
-            key[q] = e < E ? sc[q] + choice_bias[e] : -INFINITY;
-        }
-        for (int k = 0; k < top; ++k) {
-            float best = -INFINITY, best_s = 0.f;
-            int best_e = 0x7fffffff;
-#pragma unroll
-            for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q)
-                if (key[q] > best) { best = key[q]; best_e = q * IA_WAVE + lane; best_s = sc[q]; }
-#pragma unroll
-            for (int o = IA_WAVE / 2; o > 0; o >>= 1) {
-                const float ob = __shfl_xor(best, o, IA_WAVE), os = __shfl_xor(best_s, o, IA_WAVE);
-                const int oe = __shfl_xor(best_e, o, IA_WAVE);
-                if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; best_s = os; }
-            }
-#pragma unroll
-            for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q)
-                if (best_e == q * IA_WAVE + lane) key[q] = -INFINITY;
-            total += best_s;
-            if (lane == k) { mine = best_s; mine_e = best_e; }
-        }
-    } else
-    for (int k = 0; k < top; ++k) {
-        // every lane's best, then the wave's: the largest logit, of equal ones the lower index
-        float best = -INFINITY;
-        int best_e = 0x7fffffff;
-#pragma unroll
-        for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q)
-            if (z[q] > best) { best = z[q]; best_e = q * IA_WAVE + lane; }
-#pragma unroll
-        for (int o = IA_WAVE / 2; o > 0; o >>= 1) {
-            const float ob = __shfl_xor(best, o, IA_WAVE);
-            const int oe = __shfl_xor(best_e, o, IA_WAVE);
-            if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; }
-        }
-#pragma unroll
-        for (int q = 0; q < IA_MAX_EXPERTS / IA_WAVE; ++q)
-            if (best_e == q * IA_WAVE + lane) z[q] = -INFINITY;
-        const float s = score_fn == IA_SCORE_SOFTMAX ? expf(best - zmax) / denom : 1.0f / (1.0f + expf(-best));
-        total += s;
-        if (lane == k) { mine = s; mine_e = best_e; }
-    }
-    if (lane < top) {
-        sel[(long long)t * top + lane] = mine_e;
-        weight[(long long)t * top + lane] = (renorm ? mine / total : mine) * scale;
-    }
+    route_pick<IA_MAX_EXPERTS / IA_WAVE>(sel, weight, logits, t, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out);
 }
 
-// One block.  `order` [pairs]: the pairs grouped by expert; tiles: expert, first place in `order`, rows; meta[0]: tiles.
-__global__ __launch_bounds__(1024) void route_plan_kernel(int* __restrict__ order, int* __restrict__ tile_expert,
-                                                          int* __restrict__ tile_first, int* __restrict__ tile_rows,
-                                                          int* __restrict__ meta, const int* __restrict__ sel, int pairs,
-                                                          int E, int tile) {
+// The whole block.  `order` [pairs]: the pairs grouped by expert; tiles: expert, first place in `order`, rows; meta[0]: tiles.
+// sel may lie in shared memory.
+struct RoutePlan {
+    int *order, *tile_expert, *tile_first, *tile_rows, *meta;
+    int E, tile;                                   // experts with weights, rows of a tile; order null: no plan
+};
+__device__ __forceinline__ void route_plan_block(const RoutePlan& p, const int* sel, int pairs) {
+    int *order = p.order, *tile_expert = p.tile_expert, *tile_first = p.tile_first, *tile_rows = p.tile_rows, *meta = p.meta;
+    const int E = p.E, tile = p.tile;
     __shared__ int count[IA_MAX_EXPERTS], first[IA_MAX_EXPERTS], tile0[IA_MAX_EXPERTS], cursor[IA_MAX_EXPERTS];
     for (int e = threadIdx.x; e < E; e += blockDim.x) count[e] = cursor[e] = 0;
     __syncthreads();
@@ -181,15 +195,22 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(int* __restrict__ orde
     for (int p = threadIdx.x; p < pairs; p += blockDim.x)
         if (sel[p] < E) atomicAdd(&count[sel[p]], 1);
     __syncthreads();
-    if (threadIdx.x == 0) {
+    if (threadIdx.x < IA_WAVE) {                   // (running sums over the experts, 64 at a time by lane shifts)
         int at = 0, tiles = 0;
-        for (int e = 0; e < E; ++e) {
-            first[e] = at;
-            tile0[e] = tiles;
-            at += count[e];
-            tiles += (count[e] + tile - 1) / tile;
+        for (int e0 = 0; e0 < E; e0 += IA_WAVE) {
+            const int e = e0 + (int)threadIdx.x;
+            const int mine = e < E ? count[e] : 0, mine_t = (mine + tile - 1) / tile;
+            int sum = mine, sum_t = mine_t;
+#pragma unroll
+            for (int o = 1; o < IA_WAVE; o <<= 1) {
+                const int u = __shfl_up(sum, o, IA_WAVE), v = __shfl_up(sum_t, o, IA_WAVE);
+                if ((int)threadIdx.x >= o) { sum += u; sum_t += v; }
+            }
+            if (e < E) { first[e] = at + sum - mine; tile0[e] = tiles + sum_t - mine_t; }
+            at += __shfl(sum, IA_WAVE - 1, IA_WAVE);
+            tiles += __shfl(sum_t, IA_WAVE - 1, IA_WAVE);
         }
-        meta[0] = tiles;
+        if (threadIdx.x == 0) meta[0] = tiles;
     }
     __syncthreads();
     for (int e = threadIdx.x; e < E; e += blockDim.x) {
@@ -204,6 +225,90 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(int* __restrict__ orde
         const int e = sel[p];
         if (e < E) order[first[e] + atomicAdd(&cursor[e], 1)] = p;
     }
+}
+
+__global__ __launch_bounds__(1024) void route_plan_kernel(const RoutePlan p, const int* __restrict__ sel, int pairs) {
+    route_plan_block(p, sel, pairs);
+}
+
+// The router on the matrix cores, for bfloat16 rows and matrices (every product exact, the sums 32-bit) of up to 64 outputs: a
+// block of sixteen waves owns 16 tokens; wave w multiplies the steps w, w + 16, .. of 32 features, the waves' sums meet in
+// shared memory and are added in the waves' order (an order that depends on the width alone), then wave w picks for token
+// w.  A step of up to 16 tokens is one block, which then orders the pairs for the experts' products as well (`plan`): one
+// kernel where there were two.
+#define IA_RM_WAVES 16
+#define IA_RM_TOKENS 16
+template <int NT>
+__global__ __launch_bounds__(64 * IA_RM_WAVES) void route_mfma_kernel(int* __restrict__ sel, float* __restrict__ weight,
+                                                                      const bf16_t* __restrict__ h, const bf16_t* __restrict__ wr, int n,
+                                                                      int W, int E, int top, float scale, int score_fn, int renorm,
+                                                                      const float* __restrict__ choice_bias, int gates,
+                                                                      float* __restrict__ gate_out, const RoutePlan plan) {
+    extern __shared__ float rm_part[];             // [waves][tokens][16 NT]
+    __shared__ float logits[IA_RM_TOKENS][16 * NT];
+    __shared__ int chosen[IA_RM_TOKENS * IA_MAX_TOP];
+    const int t0 = blockIdx.x * IA_RM_TOKENS, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int r16 = lane & 15, G = lane >> 4;
+    const bf16_t* row = h + (long long)(t0 + r16 < n ? t0 + r16 : n - 1) * W;
+    const bf16_t* w[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) w[j] = wr + (long long)(16 * j + r16 < E ? 16 * j + r16 : E - 1) * W;
+    tm_f32x4 acc[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[j] = (tm_f32x4){0.f, 0.f, 0.f, 0.f};
+    const int steps = (W + 31) / 32;
+#pragma unroll 4
+    for (int st = wave; st < steps; st += IA_RM_WAVES) {
+        const int c = 32 * st + 8 * G;
+        const bool in = c < W;                     // (widths in steps of 8: a piece lies inside or outside as a whole)
+        const tm_u32x4 zero = {0u, 0u, 0u, 0u};
+        const tm_u32x4 x = in ? *reinterpret_cast<const tm_u32x4*>(row + c) : zero;
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            const tm_u32x4 b = in ? *reinterpret_cast<const tm_u32x4*>(w[j] + c) : zero;
+            acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(tm_bf16x8, x), __builtin_bit_cast(tm_bf16x8, b), acc[j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) rm_part[(wave * IA_RM_TOKENS + 4 * G + i) * 16 * NT + 16 * j + r16] = acc[j][i];
+    __syncthreads();
+    if (threadIdx.x < IA_RM_TOKENS * 16 * NT) {
+        float total = 0.f;
+#pragma unroll
+        for (int q = 0; q < IA_RM_WAVES; ++q) total += rm_part[q * IA_RM_TOKENS * 16 * NT + threadIdx.x];
+        (&logits[0][0])[threadIdx.x] = total;
+    }
+    __syncthreads();
+    if (t0 + wave < n)
+        route_pick<1>(sel, weight, logits[wave], t0 + wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out,
+                      chosen + wave * top);
+    if (plan.order == nullptr) return;             // (the same for all threads; the grid is one block otherwise)
+    __syncthreads();
+    route_plan_block(plan, chosen, n * top);
+}
+
+// The choice from logits that another product has left in 32-bit rows, for steps of up to 16 tokens: a wave a token, then the
+// plan.  (A router's matrix read by one compute unit takes as long as the unit's share of the memory's rate lets it; as rows
+// of a large product beside it, it is spread over the chip.)
+__global__ __launch_bounds__(64 * IA_RM_WAVES) void route_logits_kernel(int* __restrict__ sel, float* __restrict__ weight,
+                                                                        const float* __restrict__ logits, long long ld, int n, int E,
+                                                                        int top, float scale, int score_fn, int renorm,
+                                                                        const float* __restrict__ choice_bias, int gates,
+                                                                        float* __restrict__ gate_out, const RoutePlan plan) {
+    __shared__ int chosen[IA_RM_TOKENS * IA_MAX_TOP];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    if (wave < n) {
+        if (E - gates <= IA_WAVE)
+            route_pick<1>(sel, weight, logits + wave * ld, wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out,
+                          chosen + wave * top);
+        else
+            route_pick<IA_MAX_EXPERTS / IA_WAVE>(sel, weight, logits + wave * ld, wave, lane, E, top, scale, score_fn, renorm, choice_bias,
+                                                 gates, gate_out, chosen + wave * top);
+    }
+    __syncthreads();
+    route_plan_block(plan, chosen, n * top);
 }
 
 // An expert's activation over its two sums.  Clamped: g' * sigmoid(alpha g') * (u' + 1), g' = min(g, limit), u' = clamp(u,
@@ -346,17 +451,51 @@ __global__ __launch_bounds__(256) void experts_down_mfma_kernel(float* __restric
     });
 }
 
+static bool route_mfma_fits(int W, int rows, int dtype, const void* h, const void* router) {
+    return dtype == IA_BF16 && rows <= 64 && W % 8 == 0 && W >= 128 && tile_mfma_aligned(h) && tile_mfma_aligned(router);
+}
+// Whether `ia_route` makes the plan of this step itself (rows: every row of the router's matrix).
+extern "C" int ia_route_plans(int n, int W, int rows, int dtype, const void* h, const void* router) {
+    return n <= IA_RM_TOKENS && route_mfma_fits(W, rows, dtype, h, router) ? 1 : 0;
+}
+
 // choice_bias: null, or [E] 32-bit values added to the scores for the choice only (the weights are the scores themselves)
 extern "C" int ia_route(int* sel, float* weight, const void* h, const void* router, int n, int W, int E, int top,
                         float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out,
+                        int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile,
                         int dtype, hipStream_t stream) {
+    // order: null, or the plan of `ia_route_plan` is made as well (ia_route_plans(...) says for which steps)
     // E: the router's outputs that can be chosen; the matrix holds `gates` more rows behind them (see the kernel)
     IA_CHECK(gates >= 0 && (gates == 0 || gate_out != nullptr), "route: %d gate rows need a place for their values", gates);
     IA_CHECK(n >= 0 && W > 0 && E >= 1 && E + gates <= IA_MAX_EXPERTS && top >= 1 && top <= E && top <= IA_MAX_TOP,
              "route: n=%d width=%d experts=%d and %d gate rows (up to %d) top=%d (up to %d)", n, W, E, gates, IA_MAX_EXPERTS, top, IA_MAX_TOP);
     E += gates;
     IA_CHECK(score_fn == IA_SCORE_SIGMOID || score_fn == IA_SCORE_SOFTMAX, "route: unknown score function %d", score_fn);
+    IA_CHECK(order == nullptr || ia_route_plans(n, W, E, dtype, h, router), "route: this step's plan is made by a kernel of its own");
     if (n == 0) return 0;
+    if (route_mfma_fits(W, E, dtype, h, router)) {
+        RoutePlan plan;
+        plan.order = order; plan.tile_expert = tile_expert; plan.tile_first = tile_first; plan.tile_rows = tile_rows; plan.meta = meta;
+        plan.E = plan_E; plan.tile = tile;
+        const int nt = (E + 15) / 16;
+        const unsigned blocks = (unsigned)((n + IA_RM_TOKENS - 1) / IA_RM_TOKENS);
+        const size_t shm = (size_t)IA_RM_WAVES * IA_RM_TOKENS * 16 * nt * sizeof(float);
+#define IA_RM(NT)                                                                                                       \
+    do {                                                                                                                \
+        static int asked = 0;                                                                                           \
+        if (shm > 48 * 1024 && !asked) {                                                                                \
+            const hipError_t e = hipFuncSetAttribute((const void*)route_mfma_kernel<NT>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024); \
+            IA_CHECK(e == hipSuccess, "route: cannot ask for shared memory: %s", hipGetErrorString(e));                 \
+            asked = 1;                                                                                                  \
+        }                                                                                                               \
+        route_mfma_kernel<NT><<<blocks, 64 * IA_RM_WAVES, shm, stream>>>(sel, weight, (const bf16_t*)h, (const bf16_t*)router, n, W, E, top, \
+                                                                         scale, score_fn, renorm, choice_bias, gates, gate_out, plan); \
+    } while (0)
+        switch (nt) { case 1: IA_RM(1); break; case 2: IA_RM(2); break; case 3: IA_RM(3); break; default: IA_RM(4); break; }
+#undef IA_RM
+        IA_LAUNCH_CHECK("route (matrix cores)");
+        return 0;
+    }
     const bool vec = W % 8 == 0 && tile_mfma_aligned(h) && tile_mfma_aligned(router);
 #define IA_ROUTE_SW(T, V, S, WV) route_kernel<T, V, S, WV><<<n, 64 * WV, 0, stream>>>(sel, weight, (const T*)h, (const T*)router, n, W, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out)
 #define IA_ROUTE_S(T, V, S) IA_ROUTE_SW(T, V, S, IA_ROUTE_WAVES)
@@ -377,6 +516,23 @@ extern "C" int ia_route(int* sel, float* weight, const void* h, const void* rout
     return 0;
 }
 
+extern "C" int ia_route_logits(int* sel, float* weight, const float* logits, long long ld, int off, int n, int E, int top, float scale,
+                               int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order,
+                               int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, hipStream_t stream) {
+    IA_CHECK(n >= 0 && n <= IA_RM_TOKENS && E >= 1 && gates >= 0 && E + gates <= IA_MAX_EXPERTS && top >= 1 && top <= E && top <= IA_MAX_TOP &&
+             off >= 0 && off + E + gates <= ld && (gates == 0 || gate_out != nullptr) && order != nullptr,
+             "route_logits: n=%d (up to %d) experts=%d and %d gates at %d of rows of %lld, top=%d", n, IA_RM_TOKENS, E, gates, off, ld, top);
+    IA_CHECK(score_fn == IA_SCORE_SIGMOID || score_fn == IA_SCORE_SOFTMAX, "route_logits: unknown score function %d", score_fn);
+    if (n == 0) return 0;
+    RoutePlan plan;
+    plan.order = order; plan.tile_expert = tile_expert; plan.tile_first = tile_first; plan.tile_rows = tile_rows; plan.meta = meta;
+    plan.E = plan_E; plan.tile = tile;
+    route_logits_kernel<<<1, 64 * IA_RM_WAVES, 0, stream>>>(sel, weight, logits + off, ld, n, E + gates, top, scale, score_fn, renorm,
+                                                            choice_bias, gates, gate_out, plan);
+    IA_LAUNCH_CHECK("route_logits");
+    return 0;
+}
+
 // The most tiles of `tile` rows that `pairs` pairs over E experts can make: the grids of the two products.
 static int route_tiles(int pairs, int E, int tile) { return (pairs + tile - 1) / tile + (E < pairs ? E : pairs); }
 extern "C" int ia_route_tiles(int pairs, int E) { return route_tiles(pairs, E, IA_TM); }
@@ -386,7 +542,9 @@ extern "C" int ia_route_plan(int* order, int* tile_expert, int* tile_first, int*
                              int pairs, int E, int tile, hipStream_t stream) {
     IA_CHECK(pairs >= 0 && E >= 1 && E <= IA_MAX_EXPERTS && (tile == 32 || tile == 64 || tile == 128), "route_plan: pairs=%d experts=%d tile=%d",
              pairs, E, tile);
-    route_plan_kernel<<<1, 1024, 0, stream>>>(order, tile_expert, tile_first, tile_rows, meta, sel, pairs, E, tile);
+    RoutePlan p;
+    p.order = order; p.tile_expert = tile_expert; p.tile_first = tile_first; p.tile_rows = tile_rows; p.meta = meta; p.E = E; p.tile = tile;
+    route_plan_kernel<<<1, 1024, 0, stream>>>(p, sel, pairs);
     IA_LAUNCH_CHECK("route_plan");
     return 0;
 }

@@ -18,8 +18,9 @@
 // The scores P[t][s] = sum_i q_t[i] k_s[i] prod_(s<r<=t) f_r[i] are no product of two matrices, and their factors cannot be
 // split at one point of a chunk (a quotient of products would over- or underflow).  A chunk is cut into four blocks of 16
 // tokens: between blocks the factor splits at the borders, q_t (prod from its block's start) . (whole blocks between) .
-// k_s (prod to its block's end), every piece a product of numbers up to 1; inside a block the vector units form the scores
-// directly, a running product a key.
+// k_s (prod to its block's end), every piece a product of numbers up to 1.  Inside a block the same once more between its four
+// groups of 4 tokens (three products of the whole block, one a distance between groups, of which the pairs of groups at that
+// distance are kept); inside a group the vector units form the ten scores directly.
 #include "api.h"
 #include "common.h"
 
@@ -124,8 +125,13 @@ __global__ __launch_bounds__(FS_THREADS) void fading_walk_kernel(const FadingArg
 }
 
 // ---- chunks side by side ----------------------------------------------------------------------------------------------
-// Rows of a chunk into shared memory: dst[tt][i] = fn(src[(first + tt) * ld + i], i) for tt < nt, i < dim, zeros up to 64
-// rows and d16 columns.  Four pieces of a thread are asked for before the first is used.
+// The kernels below are compiled for keys of up to 16 KT entries (KT 2, 4 or 8; what lies between dim and 16 KT is zeros in
+// shared memory): with every count and every pitch a constant a wave's operand reads and products stand in one piece, where
+// tests between them left each product waiting for its own reads (a chunk's outputs 42 us alone on a compute unit).
+//
+// Rows of a chunk into shared memory: dst[tt][i] = fn(src[(first + tt) * ld + i], c[i]) for tt < nt, i < dim, zeros up to 64
+// rows and 16 KT columns.  A thread owns one 16-byte piece of a row (with `vec`; else one column) of several rows: what fn
+// needs of its columns (`consts(i)`) is read once, and every load is asked for before the first is used.
 __device__ __forceinline__ void fs_load(const float* p, float (&v)[8]) {
     const float4 q = *(const float4*)p;
     v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
@@ -140,69 +146,69 @@ __device__ __forceinline__ void fs_load(const bf16_t* p, float (&v)[8]) {
     }
 }
 
-template <typename T, typename F>
-__device__ __forceinline__ void fs_stage_rows(float* __restrict__ dst, int ld_s, const T* __restrict__ src, long long ld_g, int first,
-                                              int nt, int dim, int d16, bool vec, F fn) {
-    constexpr int E = 16 / (int)sizeof(T);
+template <typename T, int KT, typename C, typename F>
+__device__ __forceinline__ void fs_stage_rows(float* __restrict__ dst, const T* __restrict__ src, long long ld_g, int first, int nt,
+                                              int dim, bool vec, C consts, F fn) {
+    constexpr int D16 = 16 * KT, LD = D16 + 4, E = 16 / (int)sizeof(T);
     if (vec) {                                             // (dim is a multiple of E, the rows start at multiples of 16 bytes)
-        const int per_row = dim / E, total = FS_CHUNK * per_row;
-        for (int b = 0; b < total; b += 4 * FS_THREADS) {
-            float v[4][8];
+        constexpr int PPR = D16 / E, STEP = FS_THREADS / PPR, ITERS = FS_CHUNK / STEP;
+        const int piece = threadIdx.x % PPR, row0 = threadIdx.x / PPR;
+        const bool inside = piece * E < dim;
+        float v[ITERS][8];
 #pragma unroll
-            for (int it = 0; it < 4; ++it) {
-                const int idx = b + it * FS_THREADS + threadIdx.x;
-                const int tt = idx / per_row, piece = idx - tt * per_row;
-                if (idx < total && tt < nt) fs_load(src + (long long)(first + tt) * ld_g + piece * E, v[it]);
-            }
+        for (int it = 0; it < ITERS; ++it) {
+            const int tt = row0 + it * STEP;
+            fs_load(src + (long long)(first + (tt < nt ? tt : nt - 1)) * ld_g + (inside ? piece * E : 0), v[it]);
+        }
+        float2 c[E];
 #pragma unroll
-            for (int it = 0; it < 4; ++it) {
-                const int idx = b + it * FS_THREADS + threadIdx.x;
-                const int tt = idx / per_row, piece = idx - tt * per_row;
-                if (idx >= total) continue;
-                float* d = dst + tt * ld_s + piece * E;
+        for (int e = 0; e < E; ++e) c[e] = consts(inside ? piece * E + e : 0);
 #pragma unroll
-                for (int e = 0; e < E; e += 4) {
-                    float4 w = make_float4(0.f, 0.f, 0.f, 0.f);
-                    if (tt < nt) w = make_float4(fn(v[it][e], piece * E + e), fn(v[it][e + 1], piece * E + e + 1),
-                                                 fn(v[it][e + 2], piece * E + e + 2), fn(v[it][e + 3], piece * E + e + 3));
-                    *(float4*)(d + e) = w;
-                }
+        for (int it = 0; it < ITERS; ++it) {
+            const int tt = row0 + it * STEP;
+            const bool live = inside && tt < nt;
+#pragma unroll
+            for (int e = 0; e < E; e += 4) {
+                float w[4];
+#pragma unroll
+                for (int x = 0; x < 4; ++x) w[x] = live ? fn(v[it][e + x], c[e + x]) : 0.f;
+                *(float4*)(dst + tt * LD + piece * E + e) = make_float4(w[0], w[1], w[2], w[3]);
             }
         }
-        if (d16 > dim)
-            for (int e = threadIdx.x; e < FS_CHUNK * (d16 - dim); e += FS_THREADS)
-                dst[e / (d16 - dim) * ld_s + dim + e % (d16 - dim)] = 0.f;
         return;
     }
-    for (int e = threadIdx.x; e < FS_CHUNK * d16; e += FS_THREADS) {
-        const int tt = e / d16, i = e - tt * d16;
-        dst[tt * ld_s + i] = tt < nt && i < dim ? fn(ld(src + (long long)(first + tt) * ld_g + i), i) : 0.f;
-    }
+    constexpr int STEP = FS_THREADS / D16;
+    const int i = threadIdx.x % D16;
+    const float2 c = consts(i < dim ? i : 0);
+#pragma unroll 8
+    for (int tt = threadIdx.x / D16; tt < FS_CHUNK; tt += STEP)
+        dst[tt * LD + i] = tt < nt && i < dim ? fn(ld(src + (long long)(first + tt) * ld_g + i), c) : 0.f;
 }
 
-// 32 columns of v: v_s[tt][c] (zeros for tokens the chunk does not have and columns beyond vdim)
+// 32 columns of v, v_s[tt][c] (zeros for tokens the chunk does not have and columns beyond vdim): into registers, and from
+// there into shared memory.
 template <typename T>
-__device__ __forceinline__ void fs_stage_values(float* __restrict__ v_s, const T* __restrict__ v, long long ld_g, int first, int nt,
-                                                int j0, int vdim) {
+__device__ __forceinline__ void fs_fetch_values(float (&vv)[8], const T* __restrict__ v, long long ld_g, int first, int nt, int j0, int vdim) {
     const int j = j0 + (threadIdx.x & 31);
-    float vv[8];
 #pragma unroll
     for (int it = 0; it < 8; ++it) {
         const int tt = (threadIdx.x >> 5) + 8 * it;
         vv[it] = tt < nt && j < vdim ? ld(v + (long long)(first + tt) * ld_g + j) : 0.f;
     }
+}
+__device__ __forceinline__ void fs_put_values(float* __restrict__ v_s, const float (&vv)[8]) {
 #pragma unroll
     for (int it = 0; it < 8; ++it) v_s[((threadIdx.x >> 5) + 8 * it) * FS_V_LD + (threadIdx.x & 31)] = vv[it];
 }
 
 // A block of four waves owns a (chunk, head).
-template <typename T>
-__global__ __launch_bounds__(FS_THREADS) void fading_local_kernel(const FadingArgs a, int ld_s) {
+template <typename T, int KT>
+__global__ __launch_bounds__(FS_THREADS) void fading_local_kernel(const FadingArgs a) {
     extern __shared__ __attribute__((aligned(16))) float fs_shared[];
-    const int d16 = (a.dim + 15) / 16 * 16;
-    float* const k_s = fs_shared;                          // [64][ld_s]
-    float* const v_s = k_s + FS_CHUNK * ld_s;              // [64][FS_V_LD]
-    float* const m_s = v_s + FS_CHUNK * FS_V_LD;           // [4][d16]: the products of the blocks' factors
+    constexpr int D16 = 16 * KT, LD = D16 + 4, MT = (KT + 3) / 4;
+    float* const k_s = fs_shared;                          // [64][LD]
+    float* const v_s = k_s + FS_CHUNK * LD;                // [64][FS_V_LD]
+    float* const m_s = v_s + FS_CHUNK * FS_V_LD;           // [4][D16]: the products of the blocks' factors
     const int h = blockIdx.y;
     const int seq = blockIdx.z / a.chunks, c = blockIdx.z - seq * a.chunks;
     const int first = a.cu_tokens[seq] + (a.chunk0 + c) * FS_CHUNK, end = a.cu_tokens[seq + 1];
@@ -210,18 +216,21 @@ __global__ __launch_bounds__(FS_THREADS) void fading_local_kernel(const FadingAr
     const int nt = end - first < FS_CHUNK ? end - first : FS_CHUNK;
     const float *fb = a.f_bias + h * a.dim, *lo = a.lower + h * a.dim;
     const T* v = (const T*)a.proj + a.v_off + (long long)h * a.vdim;
-    fs_stage_rows<T>(k_s, ld_s, (const T*)a.proj + a.f_off + (long long)h * a.dim, a.ld, first, nt, a.dim, d16, a.vec != 0,
-                     [&](float z, int i) { return fs_open(z, fb[i], lo[i]); });
+    float vv[8];                                           // (columns of v are on their way while those before are multiplied)
+    fs_fetch_values<T>(vv, v, a.ld, first, nt, 0, a.vdim);
+    fs_stage_rows<T, KT>(k_s, (const T*)a.proj + a.f_off + (long long)h * a.dim, a.ld, first, nt, a.dim, a.vec != 0,
+                         [&](int i) { return make_float2(fb[i], lo[i]); }, [](float z, float2 g) { return fs_open(z, g.x, g.y); });
     __syncthreads();
     // (tokens the chunk does not have are zeros: their factor is 1)
-    for (int e = threadIdx.x; e < 4 * d16; e += FS_THREADS) {
-        const int sub = e / d16, i = e - sub * d16;
+#pragma unroll
+    for (int e = threadIdx.x; e < 4 * D16; e += FS_THREADS) {
+        const int sub = e / D16, i = e - sub * D16;
         float kk[FS_SUB], run = 1.f;
 #pragma unroll
-        for (int s = 0; s < FS_SUB; ++s) kk[s] = k_s[(FS_SUB * sub + s) * ld_s + i];
+        for (int s = 0; s < FS_SUB; ++s) kk[s] = k_s[(FS_SUB * sub + s) * LD + i];
 #pragma unroll
         for (int s = FS_SUB - 1; s >= 0; --s) {
-            k_s[(FS_SUB * sub + s) * ld_s + i] = kk[s] * run;
+            k_s[(FS_SUB * sub + s) * LD + i] = kk[s] * run;
             run *= 1.0f - kk[s];
         }
         m_s[e] = run;
@@ -229,42 +238,52 @@ __global__ __launch_bounds__(FS_THREADS) void fading_local_kernel(const FadingAr
     __syncthreads();
     const long long unit = (long long)blockIdx.z * a.H + h;
     for (int i = threadIdx.x; i < a.dim; i += FS_THREADS)
-        a.chunk_a[unit * a.dim + i] = m_s[i] * m_s[d16 + i] * m_s[2 * d16 + i] * m_s[3 * d16 + i];
+        a.chunk_a[unit * a.dim + i] = m_s[i] * m_s[D16 + i] * m_s[2 * D16 + i] * m_s[3 * D16 + i];
     float* const u_out = a.chunk_s + unit * a.vdim * a.dim;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int r16 = lane & 15, kq = lane >> 4;
-    const int row_tiles = d16 / 16;
+    // the wave's rows of U: tiles wave, wave + 4; their keys, to the chunk's end, stay in registers
+    float ak[MT][FS_CHUNK / 4];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int mt = wave + 4 * m, ii = 16 * (mt < KT ? mt : 0) + r16;
+        const float m1 = m_s[D16 + ii], m2 = m_s[2 * D16 + ii], m3 = m_s[3 * D16 + ii];
+        const float later[4] = {m1 * m2 * m3, m2 * m3, m3, 1.0f};
+#pragma unroll
+        for (int k4 = 0; k4 < FS_CHUNK / 4; ++k4) ak[m][k4] = k_s[(4 * k4 + kq) * LD + ii] * later[4 * k4 / FS_SUB];
+    }
     for (int j0 = 0; j0 < a.vdim; j0 += 32) {
         if (j0 > 0) __syncthreads();                       // (the columns before are used up)
-        fs_stage_values<T>(v_s, v, a.ld, first, nt, j0, a.vdim);
+        fs_put_values(v_s, vv);
+        if (j0 + 32 < a.vdim) fs_fetch_values<T>(vv, v, a.ld, first, nt, j0 + 32, a.vdim);
         __syncthreads();
-        for (int mt = wave; mt < row_tiles; mt += 4) {
-            const int ii = 16 * mt + r16;
-            const float m1 = m_s[d16 + ii], m2 = m_s[2 * d16 + ii], m3 = m_s[3 * d16 + ii];
-            const float later[4] = {m1 * m2 * m3, m2 * m3, m3, 1.0f};
-            fs_f32x4 acc[2] = {(fs_f32x4){0.f, 0.f, 0.f, 0.f}, (fs_f32x4){0.f, 0.f, 0.f, 0.f}};
-            const float* ka = k_s + kq * ld_s + ii;
-            const float* vb = v_s + kq * FS_V_LD + r16;
+        const float* vb = v_s + kq * FS_V_LD + r16;
+        fs_f32x4 acc[MT][2];
 #pragma unroll
-            for (int k0 = 0; k0 < FS_CHUNK; k0 += 4) {
-                const float av = ka[k0 * ld_s] * later[k0 / FS_SUB];
-                acc[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vb[k0 * FS_V_LD], acc[0], 0, 0, 0);
-                acc[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vb[k0 * FS_V_LD + 16], acc[1], 0, 0, 0);
+        for (int m = 0; m < MT; ++m) acc[m][0] = acc[m][1] = (fs_f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k4 = 0; k4 < FS_CHUNK / 4; ++k4) {
+            const float b0 = vb[4 * k4 * FS_V_LD], b1 = vb[4 * k4 * FS_V_LD + 16];
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+                acc[m][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak[m][k4], b0, acc[m][0], 0, 0, 0);
+                acc[m][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak[m][k4], b1, acc[m][1], 0, 0, 0);
             }
+        }
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
 #pragma unroll
             for (int c2 = 0; c2 < 2; ++c2) {
-                const int col = j0 + 16 * c2 + r16;
-                if (col >= a.vdim) continue;
-                const int i = 16 * mt + 4 * kq;
+                const int col = j0 + 16 * c2 + r16, i = 16 * (wave + 4 * m) + 4 * kq;
+                if (wave + 4 * m >= KT || col >= a.vdim) continue;
                 float* at = u_out + (long long)col * a.dim + i;
-                if (a.wide && i + 4 <= a.dim) *(float4*)at = make_float4(acc[c2][0], acc[c2][1], acc[c2][2], acc[c2][3]);
+                if (a.wide && i + 4 <= a.dim) *(float4*)at = make_float4(acc[m][c2][0], acc[m][c2][1], acc[m][c2][2], acc[m][c2][3]);
                 else {
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
-                        if (i + r < a.dim) at[r] = acc[c2][r];
+                        if (i + r < a.dim) at[r] = acc[m][c2][r];
                 }
             }
-        }
     }
 }
 
@@ -303,17 +322,18 @@ __global__ void fading_chunks_kernel(const FadingArgs a) {
 // A block of four waves owns a (chunk, head); wave w owns tokens 16 w .. 16 w + 15.  Shared memory: the queries, whose
 // rows the scores replace once a wave has its own in registers; the keys, whose place the columns of v and of the matrix
 // the chunk starts from take once the scores are formed.  NT: pairs of 16-column tiles that a wave keeps in registers.
-template <typename T, int NT>
-__global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const FadingArgs a, int ld_s, int q_floats, int k_floats) {
+template <typename T, int KT, int NT>
+__global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const FadingArgs a) {
     extern __shared__ __attribute__((aligned(16))) float fs_shared[];
-    const int d16 = (a.dim + 15) / 16 * 16;
-    float* const q_s = fs_shared;                          // [64][ld_s]
-    float* const k_s = q_s + q_floats;                     // [64][ld_s]
-    float* const m_s = k_s + k_floats;                     // [4][d16]
-    float* const p_s = q_s;                                // [64][p_ld], in the queries' rows (or rows of 68 where those are shorter)
-    const int p_ld = ld_s >= FS_CHUNK + 4 ? ld_s : FS_CHUNK + 4;
+    constexpr int D16 = 16 * KT, LD = D16 + 4, P_LD = LD >= FS_CHUNK + 4 ? LD : FS_CHUNK + 4;
+    constexpr int TILES = FS_CHUNK * FS_V_LD + 32 * LD, K_FLOATS = FS_CHUNK * LD > TILES ? FS_CHUNK * LD : TILES;
+    float* const q_s = fs_shared;                          // [64][LD]
+    float* const k_s = q_s + FS_CHUNK * P_LD;              // [64][LD]
+    float* const m_s = k_s + K_FLOATS;                     // [4][D16]: the products of the blocks' factors
+    float* const g_s = m_s + 4 * D16;                      // [4][4][D16]: of the groups of 4 tokens
+    float* const p_s = q_s;                                // [64][P_LD], in the queries' rows (or rows of 68 where those are shorter)
     float* const v_s = k_s;                                // [64][FS_V_LD]
-    float* const c_s = v_s + FS_CHUNK * FS_V_LD;           // [32][ld_s]
+    float* const c_s = v_s + FS_CHUNK * FS_V_LD;           // [32][LD]
     const int h = blockIdx.y;
     const int seq = blockIdx.z / a.chunks, c = blockIdx.z - seq * a.chunks;
     const int first = a.cu_tokens[seq] + (a.chunk0 + c) * FS_CHUNK, end = a.cu_tokens[seq + 1];
@@ -321,92 +341,142 @@ __global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const Fad
     const int nt = end - first < FS_CHUNK ? end - first : FS_CHUNK;
     const float *fb = a.f_bias + h * a.dim, *lo = a.lower + h * a.dim;
     const T* v = (const T*)a.proj + a.v_off + (long long)h * a.vdim;
-    fs_stage_rows<T>(q_s, ld_s, (const T*)a.proj + a.q_off + (long long)h * a.dim, a.ld, first, nt, a.dim, d16, a.vec != 0,
-                     [&](float u, int) { return fs_silu(u); });
-    fs_stage_rows<T>(k_s, ld_s, (const T*)a.proj + a.f_off + (long long)h * a.dim, a.ld, first, nt, a.dim, d16, a.vec != 0,
-                     [&](float z, int i) { return fs_open(z, fb[i], lo[i]); });
+    fs_stage_rows<T, KT>(q_s, (const T*)a.proj + a.q_off + (long long)h * a.dim, a.ld, first, nt, a.dim, a.vec != 0,
+                         [](int) { return make_float2(0.f, 0.f); }, [](float u, float2) { return fs_silu(u); });
+    fs_stage_rows<T, KT>(k_s, (const T*)a.proj + a.f_off + (long long)h * a.dim, a.ld, first, nt, a.dim, a.vec != 0,
+                         [&](int i) { return make_float2(fb[i], lo[i]); }, [](float z, float2 g) { return fs_open(z, g.x, g.y); });
     __syncthreads();
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int r16 = lane & 15, kq = lane >> 4;
-    // ---- the scores inside the wave's block of 16 tokens: lane (s, part) follows key s through the block, a quarter of
-    // the channels a lane, w = k_s prod_(s<r<=t) f_r
-    float inside[FS_SUB];
+    float* const q0 = q_s + FS_SUB * wave * LD;          // the wave's block of 16 tokens
+    float* const k0 = k_s + FS_SUB * wave * LD;
+    const int grp = r16 >> 2;                              // the group of 4 of row (or column) r16 of the block
+    // ---- the scores inside the groups: lane (t, part) has token t and a quarter of the channels; a running product of the
+    // factors stands with the query: near[e] is the score of token t - e (of the same group)
+    float near[4] = {0.f, 0.f, 0.f, 0.f};
     {
-        const float* q0 = q_s + FS_SUB * wave * ld_s + 4 * kq;
-        const float* k0 = k_s + FS_SUB * wave * ld_s + 4 * kq;
-        float w[FS_MAX_DIM / 16][4];
 #pragma unroll
-        for (int j = 0; j < FS_MAX_DIM / 16; ++j) {
-            if (16 * j < d16) {
-                const float4 kk = *(const float4*)(k0 + r16 * ld_s + 16 * j);
-                w[j][0] = kk.x; w[j][1] = kk.y; w[j][2] = kk.z; w[j][3] = kk.w;
-            }
-        }
+        for (int j = 0; j < KT; ++j) {
+            const float4 q4 = *(const float4*)(q0 + r16 * LD + 16 * j + 4 * kq);
+            float qf[4] = {q4.x, q4.y, q4.z, q4.w};
 #pragma unroll
-        for (int t = 0; t < FS_SUB; ++t) {
-            float acc = 0.f;
-            const bool behind = t > r16;
+            for (int e = 0; e < 4; ++e) {
+                const int s = r16 - e > 4 * grp ? r16 - e : 4 * grp;     // (beyond the group's first token: not used)
+                const float4 k4 = *(const float4*)(k0 + s * LD + 16 * j + 4 * kq);
+                const float kk[4] = {k4.x, k4.y, k4.z, k4.w};
 #pragma unroll
-            for (int j = 0; j < FS_MAX_DIM / 16; ++j) {
-                if (16 * j >= d16) continue;
-                const float4 kt = *(const float4*)(k0 + t * ld_s + 16 * j), qt = *(const float4*)(q0 + t * ld_s + 16 * j);
-                const float f[4] = {1.0f - kt.x, 1.0f - kt.y, 1.0f - kt.z, 1.0f - kt.w}, qq[4] = {qt.x, qt.y, qt.z, qt.w};
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    w[j][e] = behind ? w[j][e] * f[e] : w[j][e];
-                    acc = fmaf(qq[e], w[j][e], acc);
+                for (int x = 0; x < 4; ++x) {
+                    near[e] = fmaf(qf[x], kk[x], near[e]);
+                    qf[x] *= 1.0f - kk[x];
                 }
             }
-            acc += __shfl_xor(acc, 16, IA_WAVE);
-            acc += __shfl_xor(acc, 32, IA_WAVE);
-            inside[t] = t >= r16 ? acc : 0.f;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            near[e] += __shfl_xor(near[e], 16, IA_WAVE);
+            near[e] += __shfl_xor(near[e], 32, IA_WAVE);
         }
     }
     __builtin_amdgcn_wave_barrier();
     asm volatile("" ::: "memory");
-    // ---- the block's own products: q_t from the block's start, k_s to its end (the wave's own rows: no barrier)
-    for (int i = lane; i < d16; i += IA_WAVE) {
-        float kk[FS_SUB], run = 1.f;
+    // ---- the groups' own products: q_t from the group's start, k_s to its end (the wave's own rows: no barrier)
+    float* const g_w = g_s + 4 * wave * D16;               // [4][D16]: the products of the groups' factors
+    for (int i = lane; i < D16; i += IA_WAVE) {
+        float kk[FS_SUB], qq[FS_SUB];
 #pragma unroll
-        for (int s = 0; s < FS_SUB; ++s) kk[s] = k_s[(FS_SUB * wave + s) * ld_s + i];
+        for (int s = 0; s < FS_SUB; ++s) { kk[s] = k0[s * LD + i]; qq[s] = q0[s * LD + i]; }
 #pragma unroll
-        for (int s = 0; s < FS_SUB; ++s) {
-            run *= 1.0f - kk[s];
-            q_s[(FS_SUB * wave + s) * ld_s + i] *= run;
-        }
-        m_s[wave * d16 + i] = run;
-        run = 1.f;
+        for (int a4 = 0; a4 < 4; ++a4) {
+            float run = 1.f, back = 1.f;
 #pragma unroll
-        for (int s = FS_SUB - 1; s >= 0; --s) {
-            k_s[(FS_SUB * wave + s) * ld_s + i] = kk[s] * run;
-            run *= 1.0f - kk[s];
+            for (int e = 0; e < 4; ++e) {
+                run *= 1.0f - kk[4 * a4 + e];
+                q0[(4 * a4 + e) * LD + i] = qq[4 * a4 + e] * run;
+            }
+            g_w[a4 * D16 + i] = run;
+#pragma unroll
+            for (int e = 3; e >= 0; --e) {
+                k0[(4 * a4 + e) * LD + i] = kk[4 * a4 + e] * back;
+                back *= 1.0f - kk[4 * a4 + e];
+            }
         }
     }
-    __syncthreads();
-    float aq[FS_MAX_DIM / 4];
-#pragma unroll
-    for (int kk = 0; kk < FS_MAX_DIM / 4; ++kk) aq[kk] = 4 * kk < d16 ? q_s[(FS_SUB * wave + r16) * ld_s + 4 * kk + kq] : 0.f;
-    if (p_ld != ld_s) __syncthreads();                     // (rows of scores that do not lie in their own queries' rows)
     __builtin_amdgcn_wave_barrier();
     asm volatile("" ::: "memory");
-    float* const mine = p_s + FS_SUB * wave * p_ld;
+    // ---- between the groups of the block: row t of the queries goes back one whole group a pass, until it stands at the
+    // block's start
+    float aq[4 * KT];
 #pragma unroll
-    for (int t = 0; t < FS_SUB; ++t)
-        if ((t >> 2) == kq) mine[t * p_ld + FS_SUB * wave + r16] = inside[t];
+    for (int kk = 0; kk < 4 * KT; ++kk) aq[kk] = q0[r16 * LD + 4 * kk + kq];
+    float inside[4] = {0.f, 0.f, 0.f, 0.f};                // rows 4 kq + r, column r16
+#pragma unroll
+    for (int back = 1; back < 4; ++back) {
+        fs_f32x4 acc = (fs_f32x4){0.f, 0.f, 0.f, 0.f};
+        const float* kb = k0 + r16 * LD + kq;
+#pragma unroll
+        for (int kk = 0; kk < 4 * KT; ++kk)
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], kb[4 * kk], acc, 0, 0, 0);
+        const bool mine = kq - grp == back;                // (rows 4 kq + r are group kq, column r16 is group grp)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) inside[r] = mine ? acc[r] : inside[r];
+        const float* gb = g_w + (grp >= back ? grp - back : 0) * D16 + kq;
+#pragma unroll
+        for (int kk = 0; kk < 4 * KT; ++kk)
+            aq[kk] *= grp >= back ? gb[4 * kk] : 1.0f;
+    }
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("" ::: "memory");
+    // ---- the keys to the block's end
+    for (int i = lane; i < D16; i += IA_WAVE) {
+        const float m1 = g_w[D16 + i], m2 = g_w[2 * D16 + i], m3 = g_w[3 * D16 + i];
+        const float later[3] = {m1 * m2 * m3, m2 * m3, m3};
+#pragma unroll
+        for (int s = 0; s < 12; ++s) k0[s * LD + i] *= later[s / 4];
+        m_s[wave * D16 + i] = g_w[i] * later[0];
+    }
+    __syncthreads();                                       // (the other waves' keys and products; and their queries, which are read)
+    float* const mine = p_s + FS_SUB * wave * P_LD;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) mine[(4 * kq + r) * P_LD + FS_SUB * wave + r16] = inside[r];
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("" ::: "memory");
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+        if (kq == e && r16 - e >= 4 * grp) mine[r16 * P_LD + FS_SUB * wave + r16 - e] = near[e];
     for (int cb = wave - 1; cb >= 0; --cb) {
         fs_f32x4 acc = (fs_f32x4){0.f, 0.f, 0.f, 0.f};
-        const float* kb = k_s + (FS_SUB * cb + r16) * ld_s + kq;
+        const float* kb = k_s + (FS_SUB * cb + r16) * LD + kq;
 #pragma unroll
-        for (int kk = 0; kk < FS_MAX_DIM / 4; ++kk)
-            if (4 * kk < d16) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], kb[4 * kk], acc, 0, 0, 0);
+        for (int kk = 0; kk < 4 * KT; ++kk)
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], kb[4 * kk], acc, 0, 0, 0);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) mine[(4 * kq + r) * p_ld + FS_SUB * cb + r16] = acc[r];
+        for (int r = 0; r < 4; ++r) mine[(4 * kq + r) * P_LD + FS_SUB * cb + r16] = acc[r];
 #pragma unroll
-        for (int kk = 0; kk < FS_MAX_DIM / 4; ++kk)
-            if (4 * kk < d16) aq[kk] *= m_s[cb * d16 + 4 * kk + kq];
+        for (int kk = 0; kk < 4 * KT; ++kk)
+            aq[kk] *= m_s[cb * D16 + 4 * kk + kq];
     }
-    // ---- the outputs, 32 columns at a time
+    // ---- the outputs, 32 columns at a time; the next columns of v and of the matrix the chunk starts from are on their way
+    // in registers while these are multiplied
     const float* start = a.chunk_s + ((long long)blockIdx.z * a.H + h) * a.vdim * a.dim;
+    constexpr int per_row = D16 / 4;                       // 16-byte pieces of a column of the matrix
+    float vv[8];
+    float4 cc[KT / 2];
+    auto fetch = [&](int j0) {
+        fs_fetch_values<T>(vv, v, a.ld, first, nt, j0, a.vdim);
+        if (!a.wide) return;
+#pragma unroll
+        for (int it = 0; it < KT / 2; ++it) {
+            const int idx = threadIdx.x + it * FS_THREADS, jj = idx / per_row, piece = idx - jj * per_row;
+            cc[it] = jj < 32 && j0 + jj < a.vdim && 4 * piece < a.dim ? *(const float4*)(start + (long long)(j0 + jj) * a.dim + 4 * piece)
+                                                                      : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+    };
+    fetch(0);
+    float nw[NT][2];                                       // the norm's weights of the lane's columns
+#pragma unroll
+    for (int jt = 0; jt < NT; ++jt)
+#pragma unroll
+        for (int c2 = 0; c2 < 2; ++c2) nw[jt][c2] = a.norm_w[32 * jt + 16 * c2 + r16 < a.vdim ? 32 * jt + 16 * c2 + r16 : 0];
     fs_f32x4 acc[NT][2];
 #pragma unroll
     for (int jt = 0; jt < NT; ++jt) {
@@ -414,37 +484,37 @@ __global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const Fad
         const int j0 = 32 * jt;
         if (j0 >= a.vdim) continue;
         __syncthreads();                                   // (the keys, or the columns before, are used up)
-        fs_stage_values<T>(v_s, v, a.ld, first, nt, j0, a.vdim);
-        const int here = a.vdim - j0 < 32 ? a.vdim - j0 : 32;
+        fs_put_values(v_s, vv);
         if (a.wide) {
-            const int per_row = d16 / 4;
-            for (int idx = threadIdx.x; idx < 32 * per_row; idx += FS_THREADS) {
-                const int jj = idx / per_row, piece = idx - jj * per_row;
-                const float4 z = jj < here && 4 * piece < a.dim ? *(const float4*)(start + (long long)(j0 + jj) * a.dim + 4 * piece)
-                                                                : make_float4(0.f, 0.f, 0.f, 0.f);
-                *(float4*)(c_s + jj * ld_s + 4 * piece) = z;
+#pragma unroll
+            for (int it = 0; it < KT / 2; ++it) {
+                const int idx = threadIdx.x + it * FS_THREADS, jj = idx / per_row, piece = idx - jj * per_row;
+                if (jj < 32) *(float4*)(c_s + jj * LD + 4 * piece) = cc[it];
             }
         } else {
-            for (int e = threadIdx.x; e < 32 * d16; e += FS_THREADS) {
-                const int jj = e / d16, i = e - jj * d16;
-                c_s[jj * ld_s + i] = (jj < here && i < a.dim) ? start[(long long)(j0 + jj) * a.dim + i] : 0.f;
+            for (int e = threadIdx.x; e < 32 * D16; e += FS_THREADS) {
+                const int jj = e / D16, i = e - jj * D16;
+                c_s[jj * LD + i] = (j0 + jj < a.vdim && i < a.dim) ? start[(long long)(j0 + jj) * a.dim + i] : 0.f;
             }
         }
+        if (j0 + 32 < a.vdim) fetch(j0 + 32);
         __syncthreads();
-        const float* sb = c_s + r16 * ld_s + kq;
+        const float* sb = c_s + r16 * LD + kq;
 #pragma unroll
-        for (int kk = 0; kk < FS_MAX_DIM / 4; ++kk) {
-            if (4 * kk >= d16) continue;
+        for (int kk = 0; kk < 4 * KT; ++kk) {
             acc[jt][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], sb[4 * kk], acc[jt][0], 0, 0, 0);
-            acc[jt][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], sb[16 * ld_s + 4 * kk], acc[jt][1], 0, 0, 0);
+            acc[jt][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq[kk], sb[16 * LD + 4 * kk], acc[jt][1], 0, 0, 0);
         }
-        const float* pa = mine + r16 * p_ld + kq;
+        const float* pa = mine + r16 * P_LD + kq;
         const float* vb = v_s + kq * FS_V_LD + r16;
-#pragma unroll 4
-        for (int k0 = 0; k0 < FS_SUB * (wave + 1); k0 += 4) {
-            const float av = pa[k0];
-            acc[jt][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vb[k0 * FS_V_LD], acc[jt][0], 0, 0, 0);
-            acc[jt][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vb[k0 * FS_V_LD + 16], acc[jt][1], 0, 0, 0);
+        for (int kb = 0; kb <= wave; ++kb) {
+#pragma unroll
+            for (int k0 = 0; k0 < FS_SUB; k0 += 4) {
+                const float av = pa[FS_SUB * kb + k0];
+                const float* vk = vb + (FS_SUB * kb + k0) * FS_V_LD;
+                acc[jt][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vk[0], acc[jt][0], 0, 0, 0);
+                acc[jt][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, vk[16], acc[jt][1], 0, 0, 0);
+            }
         }
     }
     // ---- the norm over a head's columns, row by row (the 16 lanes of a row's values hold its columns)
@@ -466,12 +536,10 @@ __global__ __launch_bounds__(FS_THREADS, 2) void fading_outputs_kernel(const Fad
 #pragma unroll
         for (int c2 = 0; c2 < 2; ++c2) {
             const int col = 32 * jt + 16 * c2 + r16;
-            if (col >= a.vdim) continue;
-            const float w = a.norm_w[col];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int tt = FS_SUB * wave + 4 * kq + r;
-                if (tt < nt) st((T*)a.out + ((long long)(first + tt) * a.H + h) * a.vdim + col, acc[jt][c2][r] * rs[r] * w);
+                if (tt < nt && col < a.vdim) st((T*)a.out + ((long long)(first + tt) * a.H + h) * a.vdim + col, acc[jt][c2][r] * rs[r] * nw[jt][c2]);
             }
         }
 }
@@ -545,32 +613,38 @@ extern "C" int ia_fading_scan(void* out, float* state, long long row_floats, lon
     IA_CHECK(dim <= FS_MAX_DIM && vdim <= FS_MAX_VDIM && workspace != nullptr && norm_w != nullptr && chunks > 0,
              "fading_scan: chunks take keys up to %d, values up to %d, a workspace and the norm's weight", FS_MAX_DIM, FS_MAX_VDIM);
     IA_CHECK((long long)n_seqs * chunks <= 65535 && H <= 65535, "fading_scan: %d requests x %d chunks exceed the grid", n_seqs, chunks);
-    const int d16 = (dim + 15) / 16 * 16, ld_s = d16 + 4;
-    const int lshm = (FS_CHUNK * ld_s + FS_CHUNK * FS_V_LD + 4 * d16) * 4;
-    const int q_floats = FS_CHUNK * (ld_s > FS_CHUNK + 4 ? ld_s : FS_CHUNK + 4);
-    const int tiles = FS_CHUNK * FS_V_LD + 32 * ld_s;
-    const int k_floats = FS_CHUNK * ld_s > tiles ? FS_CHUNK * ld_s : tiles;
-    const int oshm = (q_floats + k_floats + 4 * d16) * 4;
     a.chunks = chunks;
     a.chunk_s = workspace;
     a.chunk_a = workspace + (long long)n_seqs * chunks * H * vdim * dim;
     const dim3 cgrid(1, (unsigned)H, (unsigned)(n_seqs * chunks));
     const dim3 sgrid((unsigned)(((long long)H * vdim * dim + 255) / 256), (unsigned)n_seqs);
-    static int asked[2][2];
+    static int asked[2][3][2];
     for (a.chunk0 = 0; (long long)a.chunk0 * FS_CHUNK < max_q_len; a.chunk0 += chunks) {
-        if (dtype == IA_F32) fading_local_kernel<float><<<cgrid, FS_THREADS, lshm, stream>>>(a, ld_s);
-        else fading_local_kernel<bf16_t><<<cgrid, FS_THREADS, lshm, stream>>>(a, ld_s);
-        fading_chunks_kernel<<<sgrid, 256, 0, stream>>>(a);
-#define FS_OUT(TT, NT, I, J)                                                                                              \
+#define FS_LOCAL(TT, KT)                                                                                                  \
+    fading_local_kernel<TT, KT><<<cgrid, FS_THREADS, (FS_CHUNK * (16 * KT + 4 + FS_V_LD) + 4 * 16 * KT) * 4, stream>>>(a)
+#define FS_OUT(TT, KT, NT, I, J, K)                                                                                       \
     do {                                                                                                                  \
-        if (fading_shared((const void*)fading_outputs_kernel<TT, NT>, oshm, asked[I][J], "fading_scan")) return 1;        \
-        fading_outputs_kernel<TT, NT><<<cgrid, FS_THREADS, oshm, stream>>>(a, ld_s, q_floats, k_floats);                  \
+        constexpr int ld_s = 16 * KT + 4, p_ld = ld_s >= FS_CHUNK + 4 ? ld_s : FS_CHUNK + 4;                             \
+        constexpr int tiles = FS_CHUNK * FS_V_LD + 32 * ld_s, k_floats = FS_CHUNK * ld_s > tiles ? FS_CHUNK * ld_s : tiles; \
+        constexpr int oshm = (FS_CHUNK * p_ld + k_floats + 20 * 16 * KT) * 4;                                             \
+        if (fading_shared((const void*)fading_outputs_kernel<TT, KT, NT>, oshm, asked[I][J][K], "fading_scan")) return 1;    \
+        fading_outputs_kernel<TT, KT, NT><<<cgrid, FS_THREADS, oshm, stream>>>(a);                                        \
     } while (0)
-        if (dtype == IA_F32 && vdim <= 128) FS_OUT(float, 4, 0, 0);
-        else if (dtype == IA_F32) FS_OUT(float, 8, 0, 1);
-        else if (vdim <= 128) FS_OUT(bf16_t, 4, 1, 0);
-        else FS_OUT(bf16_t, 8, 1, 1);
+#define FS_BOTH(TT, I)                                                                                                    \
+    do {                                                                                                                  \
+        if (dim <= 32) FS_LOCAL(TT, 2); else if (dim <= 64) FS_LOCAL(TT, 4); else FS_LOCAL(TT, 8);                         \
+        fading_chunks_kernel<<<sgrid, 256, 0, stream>>>(a);                                                               \
+        if (vdim <= 128) {                                                                                                \
+            if (dim <= 32) FS_OUT(TT, 2, 4, I, 0, 0); else if (dim <= 64) FS_OUT(TT, 4, 4, I, 1, 0); else FS_OUT(TT, 8, 4, I, 2, 0); \
+        } else {                                                                                                          \
+            if (dim <= 32) FS_OUT(TT, 2, 8, I, 0, 1); else if (dim <= 64) FS_OUT(TT, 4, 8, I, 1, 1); else FS_OUT(TT, 8, 8, I, 2, 1); \
+        }                                                                                                                 \
+    } while (0)
+        if (dtype == IA_F32) FS_BOTH(float, 0);
+        else FS_BOTH(bf16_t, 1);
+#undef FS_BOTH
 #undef FS_OUT
+#undef FS_LOCAL
     }
     IA_LAUNCH_CHECK("fading_scan (chunks)");
     return 0;

@@ -37,7 +37,7 @@ __device__ __forceinline__ float gb_sum_splits(const T* p, int splits, long long
     return t;
 }
 
-template <typename TY, typename TG>
+template <typename TY, typename TG, typename TX>
 __global__ __launch_bounds__(1024) void branch_step_kernel(const BranchArgs a) {
     extern __shared__ float gb_row[];            // [W]
     __shared__ float scratch[16];
@@ -59,7 +59,7 @@ __global__ __launch_bounds__(1024) void branch_step_kernel(const BranchArgs a) {
     for (int c = threadIdx.x; c < W; c += blockDim.x) {          // (a thread reads back the features it wrote)
         const float v = fmaf(gb_row[c] * rs, a.norm_w[c], a.x[at + c]);
         a.x[at + c] = v;
-        if (a.xr != nullptr) st((TG*)a.xr + at + c, v);
+        if (a.xr != nullptr) st((TX*)a.xr + at + c, v);
     }
 }
 
@@ -97,7 +97,7 @@ __device__ __forceinline__ void gb_load8_splits(const T* p, int splits, long lon
     }
 }
 
-template <typename TY, typename TG, int ITERS>
+template <typename TY, typename TG, typename TX, int ITERS>
 __global__ __launch_bounds__(1024) void branch_step_vec_kernel(const BranchArgs a) {
     __shared__ float scratch[16];
     const int W = a.W, row = blockIdx.x;
@@ -151,15 +151,15 @@ __global__ __launch_bounds__(1024) void branch_step_vec_kernel(const BranchArgs 
 #pragma unroll
         for (int i = 0; i < 8; ++i) v[it][i] = fmaf(v[it][i] * rs, wv[it][i], xv[it][i]);
         gb_store8(a.x + at + c, v[it]);
-        if (a.xr != nullptr) gb_store8((TG*)a.xr + at + c, v[it]);
+        if (a.xr != nullptr) gb_store8((TX*)a.xr + at + c, v[it]);
     }
 }
 
-// y_dtype: precision of y1 and y3; g_dtype: of the gate's rows and of xr.  0 float32, 1 bfloat16.
+// y_dtype: precision of y1 and y3; g_dtype: of the gate's rows; x_dtype: of xr.  0 float32, 1 bfloat16.
 extern "C" int ia_branch_step(float* x, const void* y1, const void* y3, int y1_splits, int y3_splits, const float* y3_scale,
                               const float* routed, const float* routed_w, int top, const void* gate, long long g_ld, int g_off,
                               const float* gate_b, const float* norm_w, float eps, void* xr, int n, int W, int y_dtype,
-                              int g_dtype, hipStream_t stream) {
+                              int g_dtype, int x_dtype, hipStream_t stream) {
     IA_CHECK(n >= 0 && W > 0 && x != nullptr && norm_w != nullptr, "branch_step: n=%d width=%d, the stream and the norm's weight", n, W);
     IA_CHECK((size_t)W * sizeof(float) <= 60 * 1024, "branch_step: width %d does not fit shared memory", W);
     IA_CHECK(y1 != nullptr || routed != nullptr || y3 != nullptr, "branch_step: nothing to add");
@@ -169,7 +169,8 @@ extern "C" int ia_branch_step(float* x, const void* y1, const void* y3, int y1_s
              W, g_off, g_ld);
     IA_CHECK(y1_splits >= 1 && y3_splits >= 1 && ((y1_splits == 1 && y3_splits == 1) || y_dtype == IA_F32),
              "branch_step: outputs in %d and %d splits are 32-bit", y1_splits, y3_splits);
-    IA_CHECK((y_dtype == IA_F32 || y_dtype == IA_BF16) && (g_dtype == IA_F32 || g_dtype == IA_BF16), "branch_step: unknown dtype");
+    IA_CHECK((y_dtype == IA_F32 || y_dtype == IA_BF16) && (g_dtype == IA_F32 || g_dtype == IA_BF16) &&
+             (x_dtype == IA_F32 || x_dtype == IA_BF16), "branch_step: unknown dtype");
     if (n == 0) return 0;
     BranchArgs a;
     a.x = x; a.y1 = y1; a.y3 = y3; a.y1_splits = y1_splits; a.y3_splits = y3_splits; a.split_stride = (long long)n * W;
@@ -177,19 +178,25 @@ extern "C" int ia_branch_step(float* x, const void* y1, const void* y3, int y1_s
     a.gate_b = gate_b; a.norm_w = norm_w; a.eps = eps; a.xr = xr; a.W = W;
     const uintptr_t ptrs = (uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y3 | (uintptr_t)routed | (uintptr_t)gate | (uintptr_t)gate_b |
                            (uintptr_t)norm_w | (uintptr_t)xr;
-#define GB_TYPES(CALL)                                                     \
-    do {                                                                   \
-        if (y_dtype == IA_F32 && g_dtype == IA_F32) { CALL(float, float); } \
-        else if (y_dtype == IA_F32) { CALL(float, bf16_t); }               \
-        else if (g_dtype == IA_F32) { CALL(bf16_t, float); }               \
-        else { CALL(bf16_t, bf16_t); }                                     \
+#define GB_TYPES_X(CALL, TX)                                                    \
+    do {                                                                        \
+        if (y_dtype == IA_F32 && g_dtype == IA_F32) { CALL(float, float, TX); } \
+        else if (y_dtype == IA_F32) { CALL(float, bf16_t, TX); }                \
+        else if (g_dtype == IA_F32) { CALL(bf16_t, float, TX); }                \
+        else { CALL(bf16_t, bf16_t, TX); }                                      \
     } while (0)
-    if (W % 8 == 0 && (gate == nullptr || (g_ld % 8 == 0 && g_off % 8 == 0)) && (ptrs & 15) == 0 && W <= 8 * GB_VEC_ITERS * 1024) {
+#define GB_TYPES(CALL)                                                          \
+    do {                                                                        \
+        if (x_dtype == IA_F32) GB_TYPES_X(CALL, float);                         \
+        else GB_TYPES_X(CALL, bf16_t);                                          \
+    } while (0)
+    const int g_per = g_dtype == IA_F32 ? 4 : 8;
+    if (W % 8 == 0 && (gate == nullptr || (g_ld % g_per == 0 && g_off % g_per == 0)) && (ptrs & 15) == 0 && W <= 8 * GB_VEC_ITERS * 1024) {
         // a piece of eight a thread up to 512 threads, then more rounds
         const int pieces = W / 8;
-#define GB_VEC1(TY, TG) branch_step_vec_kernel<TY, TG, 1><<<n, (pieces + 63) / 64 * 64, 0, stream>>>(a)
-#define GB_VEC2(TY, TG) branch_step_vec_kernel<TY, TG, 2><<<n, (pieces + 127) / 128 * 64, 0, stream>>>(a)
-#define GB_VEC4(TY, TG) branch_step_vec_kernel<TY, TG, 4><<<n, (pieces + 255) / 256 * 64, 0, stream>>>(a)
+#define GB_VEC1(TY, TG, TX) branch_step_vec_kernel<TY, TG, TX, 1><<<n, (pieces + 63) / 64 * 64, 0, stream>>>(a)
+#define GB_VEC2(TY, TG, TX) branch_step_vec_kernel<TY, TG, TX, 2><<<n, (pieces + 127) / 128 * 64, 0, stream>>>(a)
+#define GB_VEC4(TY, TG, TX) branch_step_vec_kernel<TY, TG, TX, 4><<<n, (pieces + 255) / 256 * 64, 0, stream>>>(a)
         if (pieces <= 512) GB_TYPES(GB_VEC1);
         else if (pieces <= 1024) GB_TYPES(GB_VEC2);
         else GB_TYPES(GB_VEC4);
@@ -201,10 +208,11 @@ extern "C" int ia_branch_step(float* x, const void* y1, const void* y3, int y1_s
     }
     const int threads = W >= 4096 ? 1024 : W >= 1024 ? 512 : W >= 512 ? 256 : 128;
     const size_t shm = (size_t)W * sizeof(float);
-#define GB_PLAIN(TY, TG) branch_step_kernel<TY, TG><<<n, threads, shm, stream>>>(a)
+#define GB_PLAIN(TY, TG, TX) branch_step_kernel<TY, TG, TX><<<n, threads, shm, stream>>>(a)
     GB_TYPES(GB_PLAIN);
 #undef GB_PLAIN
 #undef GB_TYPES
+#undef GB_TYPES_X
     IA_LAUNCH_CHECK("branch_step");
     return 0;
 }

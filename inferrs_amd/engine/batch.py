@@ -55,6 +55,7 @@ class StepContext:
     side_rows: Any = None                   # the rows of an embedding's second table for the step's tokens, which layers take slices of
     normed: Any = None                      # (norm part, rows): the stream's rows through that norm already, left by the block before
     beside: Any = None                      # (rows, offset): the product of the weights that a block has laid beside a mixer's own projection
+    router_logits: Any = None               # (32-bit rows, offset): the logits of the next feed-forward's router, from a product that its matrix joined
     post_rows: Any = None                   # a 32-bit stream's rows once more in the products' precision, where a part has them already (the embedding, a block's last kernel)
     _tables: Dict[Any, Any] = field(default_factory=dict)
 

@@ -76,7 +76,7 @@ class _Timed:
         fn = getattr(self._lib, name)
         if KernelTimer.active is None or not name.startswith("ia_") or name.endswith(("_workspace", "_blocks", "_block_rows",
                                                                                       "_error", "_version", "_capacity", "_top",
-                                                                                      "_splits", "_tune", "_target", "_counters", "_fills", "_plan")):
+                                                                                      "_splits", "_tune", "_target", "_counters", "_fills", "_plan", "_plans")):
             return fn
         timer = KernelTimer.active
         return lambda *args: timer.call(name[3:], fn, *args)

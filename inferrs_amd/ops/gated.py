@@ -15,7 +15,8 @@ from .mix import MAX_TOP
 FADING_MAX_DIM = 512              # rows of a head's matrix that the walk takes
 FADING_CHUNK_DIM, FADING_CHUNK_VDIM = 128, 256      # keys and values that the chunks take
 FADING_CHUNK = 64                 # tokens of a chunk when long portions run in chunks side by side
-FADING_CHUNKS_FROM = 128          # steps whose longest portion has more tokens than this run in chunks
+FADING_CHUNKS_FROM = 80           # steps whose longest portion has more tokens than this run in chunks (16 heads of 128 x 128: a walk takes
+                                  # 10 us and 0.5 us a token, the three kernels of the chunks 45 us up to 128 tokens)
 FADING_WORKSPACE_FLOATS = 1 << 28     # a pass over the chunks takes no more than this (1 GiB): more passes beyond
 
 
@@ -67,14 +68,13 @@ def branch_step(x: torch.Tensor, *, y=None, routed: Optional[torch.Tensor] = Non
         if not gate.is_cuda or gate.dim() != 2 or gate.stride(1) != 1 or gate.shape[0] != n or gate_bias is None or gate_bias.numel() != W:
             raise KernelError(f"branch_step: a gate {tuple(gate.shape)} with its bias does not fit the stream [{n}, {W}]")
         g_ld = gate.stride(0) if n > 1 else gate.shape[1]
-        if gate_off < 0 or gate_off + W > gate.shape[1] or (x_dtype is not None and x_dtype != gate.dtype):
-            raise KernelError(f"branch_step: a gate of {W} features at {gate_off} of {gate.shape[1]}, in the precision of the result")
-    out_dtype = x_dtype if x_dtype is not None else (gate.dtype if gate is not None else torch.float32)
+        if gate_off < 0 or gate_off + W > gate.shape[1]:
+            raise KernelError(f"branch_step: a gate of {W} features at {gate_off} of {gate.shape[1]}")
     xr = torch.empty((n, W), dtype=x_dtype, device=x.device) if x_dtype is not None else None
     _check(library().ia_branch_step(
         _p(x), _p(y), _p(y3), splits[0], splits[1], _p(y3_scale), _p(routed), _p(routed_weights), top,
         gate.data_ptr() if gate is not None else None, g_ld, gate_off, _p(gate_bias), _p(weight), ctypes.c_float(eps), _p(xr),
-        n, W, _dt(given[0]) if given else 0, _DT[out_dtype], _stream()))
+        n, W, _dt(given[0]) if given else 0, _dt(gate) if gate is not None else 0, _DT[x_dtype] if x_dtype is not None else 0, _stream()))
     return xr
 
 

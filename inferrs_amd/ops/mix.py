@@ -223,14 +223,31 @@ def rglru_scan(u: torch.Tensor, z: torch.Tensor, proj: torch.Tensor, *, branch_o
 
 # ---- routed experts -----------------------------------------------------------------------------
 
+class ExpertPlan:
+    """Where the (row, expert) pairs of a step go in the experts' products: the pairs ordered by expert and a table of row
+    tiles, on the device.  `done`: filled already (`route` may do that; else `experts_forward` does)."""
+    __slots__ = ("pairs", "experts", "tile", "parts", "done")
+
+    def __init__(self, rows: int, top: int, experts: int, tiled: bool, device):
+        pairs = rows * top
+        tiles = -(-pairs // ROW_TILE) + min(experts, pairs)
+        # many rows an expert: the matrix cores' large tiles (64 rows x 128 features)
+        self.tile = LARGE_TILE if tiled and pairs >= LARGE_TILE_FROM * LARGE_TILE * experts else ROW_TILE
+        self.pairs, self.experts, self.done = pairs, experts, False
+        words = torch.empty((pairs + 3 * tiles + 1,), dtype=torch.int32, device=device)
+        self.parts = (words[:pairs], words[pairs:pairs + tiles], words[pairs + tiles:pairs + 2 * tiles],
+                      words[pairs + 2 * tiles:pairs + 3 * tiles], words[pairs + 3 * tiles:])     # order, expert, first, rows; tiles
+
+
 def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, score: str = "sigmoid",
-          renormalize: bool = False, choice_bias: Optional[torch.Tensor] = None, gates: int = 0):
+          renormalize: bool = False, choice_bias: Optional[torch.Tensor] = None, gates: int = 0, plan: Optional["ExpertPlan"] = None):
     """Router logits in 32-bit (router [E, width] in the precision of h; every logit is a sum of 32-bit
     multiply-adds in an order that the width alone decides), the `top` experts by score for every row:
     (experts int32 [n, top] best first, weights float32 [n, top] = score * scale).  `choice_bias` [E] (32-bit):
     the choice goes by score + bias, the weights stay the scores.  `gates`: the last `gates` rows of `router` are no
     experts: they take no part in the choice, and the sigmoids of their logits (formed like the others, in 32-bit) come
-    back as a third result, float32 [n, gates]."""
+    back as a third result, float32 [n, gates].  `plan`: an `ExpertPlan` for this step; where the kernel can (bfloat16, up to 16
+    rows and 64 outputs: one block sees every choice) it orders the pairs for the experts' products on the way."""
     _dev(h, router, choice_bias); _f32(choice_bias, "choice_bias")
     n, W = h.shape
     E = router.shape[0] - gates
@@ -245,9 +262,37 @@ def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, score: 
     sel = torch.empty((n, top), dtype=torch.int32, device=h.device)
     weight = torch.empty((n, top), dtype=torch.float32, device=h.device)
     gate_out = torch.empty((n, gates), dtype=torch.float32, device=h.device) if gates else None
+    made = (None,) * 5 + (0, 0)
+    if plan is not None and library().ia_route_plans(n, W, E + gates, _dt(h), _p(h), _p(router)):
+        if plan.pairs != n * top:
+            raise KernelError(f"route: a plan for {plan.pairs} pairs in a step of {n} rows, {top} experts each")
+        made = tuple(_p(x) for x in plan.parts) + (plan.experts, plan.tile)
+        plan.done = True
     _check(library().ia_route(_p(sel), _p(weight), _p(h), _p(router), n, W, E, top, ctypes.c_float(scale),
-                              SCORE_FUNCTIONS[score], int(renormalize), _p(choice_bias), gates, _p(gate_out), _dt(h), _stream()))
+                              SCORE_FUNCTIONS[score], int(renormalize), _p(choice_bias), gates, _p(gate_out), *made, _dt(h), _stream()))
     return (sel, weight, gate_out) if gates else (sel, weight)
+
+
+ROUTE_LOGITS_ROWS = 16        # rows of a step whose router's logits may come with another product (`route_logits`)
+
+
+def route_logits(rows: torch.Tensor, off: int, experts: int, top: int, scale: float, score: str, renormalize: bool,
+                 choice_bias: Optional[torch.Tensor], gates: int, plan: ExpertPlan):
+    """`route` from logits that a product beside the router's matrix has left: 32-bit rows [n, ..] (up to `ROUTE_LOGITS_ROWS`),
+    the experts' logits from column `off` on, those of the `gates` behind them.  The plan is made as well.  Returns
+    (experts, weights, gates or None)."""
+    _dev(rows, choice_bias); _f32(rows, "logits"); _f32(choice_bias, "choice_bias")
+    n, ld = rows.shape
+    if n > ROUTE_LOGITS_ROWS or off < 0 or off + experts + gates > ld or plan.pairs != n * top or score not in SCORE_FUNCTIONS:
+        raise KernelError(f"route_logits: logits {tuple(rows.shape)} at {off} for {experts} experts and {gates} gates, a plan of {plan.pairs} pairs")
+    sel = torch.empty((n, top), dtype=torch.int32, device=rows.device)
+    weight = torch.empty((n, top), dtype=torch.float32, device=rows.device)
+    gate_out = torch.empty((n, gates), dtype=torch.float32, device=rows.device) if gates else None
+    _check(library().ia_route_logits(_p(sel), _p(weight), _p(rows), ld, off, n, experts, top, ctypes.c_float(scale), SCORE_FUNCTIONS[score],
+                                     int(renormalize), _p(choice_bias), gates, _p(gate_out), *(_p(x) for x in plan.parts), plan.experts,
+                                     plan.tile, _stream()))
+    plan.done = True
+    return sel, weight, gate_out
 
 
 def tile_weights(w: torch.Tensor) -> torch.Tensor:
@@ -267,7 +312,7 @@ def experts_tiled_fits(dtype: torch.dtype, width: int, ff: int) -> bool:
 
 def experts_forward(h: torch.Tensor, sel: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
                     limit: float, alpha: float, ff: Optional[int] = None, in_weight: Optional[torch.Tensor] = None,
-                    activation: str = "clamped") -> torch.Tensor:
+                    activation: str = "clamped", plan: Optional[ExpertPlan] = None) -> torch.Tensor:
     """The chosen experts of every row: w_gate_up [E, 2 ff, width] (gate rows, then up rows), w_down [E, width, ff],
     or both as tiles (`tile_weights` of [E, 2, ff, width] and of [E, width, ff]; then `ff` is given);
     act = g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit); with `activation`
@@ -297,14 +342,16 @@ def experts_forward(h: torch.Tensor, sel: torch.Tensor, w_gate_up: torch.Tensor,
     if sel.shape[0] != n or E > MAX_EXPERTS:
         raise KernelError(f"experts: {tuple(sel.shape)} choices for {n} rows, {E} experts")
     pairs = n * top
-    tiles = -(-pairs // ROW_TILE) + min(E, pairs)
-    # many rows an expert: the matrix cores' large tiles (64 rows x 128 features)
-    tile = LARGE_TILE if tiled and pairs >= LARGE_TILE_FROM * LARGE_TILE * E else ROW_TILE
+    if plan is None:
+        plan = ExpertPlan(n, top, E, tiled, h.device)
+    elif plan.pairs != pairs or plan.experts != E or (plan.tile != ROW_TILE and not tiled):
+        raise KernelError(f"experts: a plan for {plan.pairs} pairs over {plan.experts} experts, not {pairs} over {E}")
+    tile = plan.tile
+    order, t_exp, t_first, t_rows, meta = plan.parts
     lib = library()
-    plan = torch.empty((pairs + 3 * tiles + 1,), dtype=torch.int32, device=h.device)
-    order, t_exp, t_first, t_rows, meta = (plan[:pairs], plan[pairs:pairs + tiles], plan[pairs + tiles:pairs + 2 * tiles],
-                                           plan[pairs + 2 * tiles:pairs + 3 * tiles], plan[pairs + 3 * tiles:])
-    _check(lib.ia_route_plan(_p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta), _p(sel), pairs, E, tile, _stream()))
+    if not plan.done:
+        _check(lib.ia_route_plan(_p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta), _p(sel), pairs, E, tile, _stream()))
+        plan.done = True
     act = torch.empty((pairs, ff), dtype=h.dtype, device=h.device)
     _check(lib.ia_experts_gate_up(_p(act), _p(h), _p(w_gate_up), _p(order), _p(t_exp), _p(t_first), _p(t_rows), _p(meta),
                                   pairs, E, top, W, ff, ctypes.c_float(limit), ctypes.c_float(alpha), EXPERT_ACTIVATIONS[activation], tile, int(tiled),

@@ -53,6 +53,7 @@ class RoutedRows:
 @register_ffn("routed_experts")
 class RoutedExperts(FeedForward):
     graph_safe = True
+    takes_logits = True           # steps of a few rows: the router's logits may come in `ctx.router_logits` = (32-bit rows, offset)
 
     @classmethod
     def tensors(cls, spec: RoutedExpertsSpec) -> Dict[str, TensorSpec]:
@@ -113,13 +114,19 @@ class RoutedExperts(FeedForward):
         if hasattr(h, "materialize"):
             h = h.materialize()
         gate = None
-        if s.shared_gate:
-            sel, weights, gate = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, gates=1)
+        plan = ops.mix.ExpertPlan(h.shape[0], s.top, s.experts, self.tiled, h.device)
+        logits = getattr(ctx, "router_logits", None)
+        if logits is not None:                       # (a block has laid the router's matrix beside one of its own)
+            ctx.router_logits = None
+            sel, weights, gate = ops.mix.route_logits(logits[0], logits[1], s.experts + s.identity, s.top, s.scale, s.score, s.renormalize,
+                                                      self.correction, int(s.shared_gate), plan)
+        elif s.shared_gate:
+            sel, weights, gate = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, gates=1, plan=plan)
         else:
-            sel, weights = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction)
+            sel, weights = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, plan=plan)
         rows = ops.experts_forward(h, sel, self.gate_up, self.down, s.limit, s.alpha,
                                    ff=s.intermediate if self.tiled else None,
-                                   in_weight=weights if s.weight_on_input else None, activation=s.activation)
+                                   in_weight=weights if s.weight_on_input else None, activation=s.activation, plan=plan)
         extra = self.shared.forward(ctx, h) if self.shared is not None else None
         if s.weight_on_input:
             weights = None

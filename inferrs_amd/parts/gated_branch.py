@@ -10,7 +10,10 @@ still split along its k, the weighted rows of routed experts, a shared expert's 
 and adds the result, and writes both arrays.  A block leaves nothing to be added.
 
 The mixer's gate reads what the mixer's own projection reads: a mixer with `lays_beside` takes the gate's matrix into its
-product (`lay_beside`, once, when the block is built) and leaves (rows, offset) in `ctx.beside` when it runs.
+product (`lay_beside`, once, when the block is built) and leaves (rows, offset) in `ctx.beside` when it runs.  The feed-forward's
+gate and a router's matrix read the same rows too: steps of a few rows form gate and logits in one product with 32-bit
+results (`ctx.router_logits`), longer ones apart (the gate in the products' precision, the logits in 32-bit by the
+router's own kernel).
 """
 from __future__ import annotations
 
@@ -81,7 +84,17 @@ class GatedBranchBlock(BlockBase):
             else:
                 self.gate_mixer = Linear([tensors[names[0]]], dtype, device)
         if len(names) > 1:
-            self.gate_bias_ffn, self.gate_ffn = biases[1], Linear([tensors[names[1]]], dtype, device)
+            self.gate_bias_ffn = biases[1]
+            weights = [Linear([tensors[names[1]]], dtype, device).weight]
+            if getattr(self.ffn, "takes_logits", False) and dtype == torch.bfloat16:
+                # the router's rows behind the gate's: steps of a few rows form both in one product with 32-bit results
+                # (padded with rows of zeros: the result's rows then start at multiples of 16 bytes)
+                pad = -(weights[0].shape[0] + self.ffn.router.shape[0]) % 8
+                weights += [self.ffn.router, torch.zeros((pad, weights[0].shape[1]), dtype=dtype, device=weights[0].device)]
+            self.gate_ffn = torch.cat(weights, dim=0).contiguous()
+            self.gate_rows = weights[0].shape[0]
+            if len(weights) > 1:
+                self.ffn.router = self.gate_ffn[self.gate_rows:self.gate_rows + self.ffn.router.shape[0]]
 
     def parts(self):
         return [self, self.mixer, self.ffn, *self.norms, getattr(self.mixer, "position", None),
@@ -121,6 +134,18 @@ class GatedBranchBlock(BlockBase):
         xr = ops.branch_step(x, weight=norm.weight, eps=norm.eps, x_dtype=None if self.dtype == torch.float32 else self.dtype, **adds)
         return x if xr is None else xr
 
+    def _ffn_gate(self, ctx, h):
+        """The feed-forward's gate; in steps of a few rows the router's logits with it (`ctx.router_logits`)."""
+        ctx.router_logits = None
+        if self.gate_ffn is None:
+            return None
+        if self.gate_ffn.shape[0] > self.gate_rows:
+            if h.shape[0] <= min(ops.mix.ROUTE_LOGITS_ROWS, ops.SKINNY_MAX_ROWS) and ops.skinny_fits(h, self.gate_ffn):
+                rows = ops.linear(h, self.gate_ffn, torch.float32)
+                ctx.router_logits = (rows, self.gate_rows)
+                return rows, 0
+        return ops.linear(h, self.gate_ffn[:self.gate_rows]), 0
+
     def forward(self, ctx, x: torch.Tensor, pending, cache, next_norm=None) -> Tuple[torch.Tensor, object]:
         if x.dim() != 2 or x.dtype != torch.float32:
             raise SpecError(f"gated_branch: the block takes a 32-bit stream [tokens, width], got {tuple(x.shape)} {x.dtype}")
@@ -139,7 +164,7 @@ class GatedBranchBlock(BlockBase):
             gate = (self.gate_mixer(h), 0)
         h = self._close(x, out, self.norms[0], gate, self.gate_bias_mixer)
         if self.ffn is not None:
-            gate = None if self.gate_ffn is None else (self.gate_ffn(h), 0)
+            gate = self._ffn_gate(ctx, h)
             h = self._close(x, self.ffn.forward(ctx, h), self.norms[1], gate, self.gate_bias_ffn)
         ctx.beside = None
         ctx.post_rows = h

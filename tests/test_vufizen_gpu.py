@@ -368,6 +368,28 @@ def test_router_softmax_over_the_chosen(E, top, W, dtype):
         np.testing.assert_allclose(sg.cpu().numpy(), torch.sigmoid(h.double() @ gate.double().T).numpy(), rtol=1e-4, atol=1e-6)
 
 
+@pytest.mark.parametrize("E,top,n", [(12, 4, 16), (33, 1, 5), (63, 8, 1), (2, 2, 9)])
+def test_the_router_makes_the_plan_of_a_short_step(E, top, n):
+    """The pairs ordered by expert and the table of row tiles, made on the way by the router's kernel: what the kernel of its
+    own makes of the same choices (the pairs of an expert in any order)."""
+    from inferrs_amd import ops
+    g = torch.Generator().manual_seed(E)
+    h, router = torch.randn(n, 256, generator=g).bfloat16(), torch.randn(E + 1, 256, generator=g).bfloat16()
+    made = ops.mix.ExpertPlan(n, top, E, True, torch.device("cuda"))
+    sel, weight, gate = ops.route(dev(h), dev(router), top, 1.0, "softmax", True, None, gates=1, plan=made)
+    assert made.done
+    own = ops.mix.ExpertPlan(n, top, E, True, torch.device("cuda"))
+    order, expert, first, rows, meta = own.parts
+    ops._check(ops.library().ia_route_plan(*(ops._p(t) for t in own.parts), ops._p(sel), n * top, E, own.tile, ops._stream()))
+    tiles = int(meta[0])
+    assert int(made.parts[4][0]) == tiles
+    assert all(torch.equal(made.parts[i][:tiles], own.parts[i][:tiles]) for i in (1, 2, 3))
+    flat = sel.flatten().cpu()
+    for plan in (made, own):
+        o = plan.parts[0].cpu().long()
+        assert sorted(o.tolist()) == list(range(n * top)) and torch.equal(flat[o], torch.sort(flat).values)
+
+
 @BOTH
 @pytest.mark.parametrize("E,top,W,ff", [(5, 2, 48, 24), (3, 3, 50, 30), (6, 2, 64, 32), (10, 1, 384, 48)])
 def test_experts_without_limits(E, top, W, ff, dtype):
