@@ -349,7 +349,7 @@ def test_fading_recurrence_remembers_one_token():
 # ---- the router and the experts ---------------------------------------------------------------------------------
 
 @BOTH
-@pytest.mark.parametrize("E,top,W", [(5, 2, 48), (1, 1, 64), (3, 3, 50), (70, 6, 136), (12, 4, 256)])
+@pytest.mark.parametrize("E,top,W", [(5, 2, 48), (1, 1, 64), (3, 3, 50), (70, 6, 136), (11, 3, 272)])
 def test_router_softmax_over_the_chosen(E, top, W, dtype):
     from inferrs_amd import ops
     g = torch.Generator().manual_seed(E * W)
@@ -368,7 +368,7 @@ def test_router_softmax_over_the_chosen(E, top, W, dtype):
         np.testing.assert_allclose(sg.cpu().numpy(), torch.sigmoid(h.double() @ gate.double().T).numpy(), rtol=1e-4, atol=1e-6)
 
 
-@pytest.mark.parametrize("E,top,n", [(12, 4, 16), (33, 1, 5), (63, 8, 1), (2, 2, 9)])
+@pytest.mark.parametrize("E,top,n", [(11, 5, 16), (33, 1, 5), (63, 8, 1), (2, 2, 9)])
 def test_the_router_makes_the_plan_of_a_short_step(E, top, n):
     """The pairs ordered by expert and the table of row tiles, made on the way by the router's kernel: what the kernel of its
     own makes of the same choices (the pairs of an expert in any order)."""
