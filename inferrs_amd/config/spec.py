@@ -233,8 +233,8 @@ class LatentAttentionSpec:
 
 @dataclass(frozen=True)
 class DifferentialAttentionSpec:
-    """Softmax attention of two maps a head over shared values, the second taken off the first: a head's queries (and a key head's keys) are
-    2 * head_dim rows, map 1's before map 2's; lambda = exp(lq1 . lk1) - exp(lq2 . lk2) +
+    """Softmax attention of two maps a head over shared values, the second taken off the first: a head's queries (and a
+    key head's keys) are 2 * head_dim rows, map 1's before map 2's; lambda = exp(lq1 . lk1) - exp(lq2 . lk2) +
     `diff`, one number a layer; o = a1 - lambda a2, brought to unit root mean square a head (`norm_eps`), times 1 -
     `diff`.  Ahead of the maps q, k and v pass a causal convolution of `conv` taps a channel (tensors "q.conv", "k.conv",
     "v.conv" [channels, conv], no bias), q and k then an RMS norm a map (weights "q.norm", "k.norm" [head_dim]) and the turn
