@@ -38,10 +38,11 @@ def _fail() -> None:
 class _Handle:
     """Owns one native cache manager."""
 
-    def __init__(self, page_size: int, max_seqs: int, windows: Sequence[int], num_pages: Sequence[int]):
+    def __init__(self, page_size: int, max_seqs: int, windows: Sequence[int], keep_first: Sequence[int],
+                 num_pages: Sequence[int]):
         self.lib = native.runtime()
         self.ptr = self.lib.iar_cache_create(page_size, max_seqs, len(windows), native.ints(list(windows)),
-                                             native.ints(list(num_pages)))
+                                             native.ints(list(keep_first)), native.ints(list(num_pages)))
         if not self.ptr:
             _fail()
 
@@ -59,7 +60,7 @@ class PagePool:
         if _handle is None:
             if num_pages < 0:
                 raise CacheError(f"num_pages must be >= 0, got {num_pages}")
-            _handle = _Handle(1, 1, [-1], [num_pages])
+            _handle = _Handle(1, 1, [-1], [0], [num_pages])
         self._h, self._g = _handle, _group
 
     @property
@@ -89,7 +90,7 @@ class SlotPool:
     """Ids 0..n-1 for per-request state of fixed size; lowest free id first."""
 
     def __init__(self, num_slots: int, _handle: Optional[_Handle] = None):
-        self._h = _handle or _Handle(1, num_slots, [], [])
+        self._h = _handle or _Handle(1, num_slots, [], [], [])
         self.num_slots = num_slots
 
     @property
@@ -248,7 +249,7 @@ class CacheManager:
         if len(num_pages) != len(grouped):
             raise CacheError(f"{len(grouped)} cache groups but {len(num_pages)} page counts")
         windows = [-1 if need.window is None else need.window for need, _ in grouped]
-        self._h = _Handle(page_size, max_seqs, windows, list(num_pages))
+        self._h = _Handle(page_size, max_seqs, windows, [need.keep_first for need, _ in grouped], list(num_pages))
         self.names = native.KeyTable()
         self.groups: List[GroupInfo] = [GroupInfo(i, need, layers, PagePool(0, self._h, i))
                                         for i, (need, layers) in enumerate(grouped)]

@@ -22,6 +22,7 @@ from .buketar import BuketarConfig
 from .fisanex import FisanexConfig
 from .ligizen import LigizenConfig
 from .lofudra import LofudraConfig
+from .lumedra import LumedraConfig
 from .qwen3 import Qwen3Config
 from .spec import ModelSpec
 from .vufizen import VufizenConfig
@@ -78,3 +79,4 @@ register_architecture(LofudraConfig)
 register_architecture(FisanexConfig)
 register_architecture(LigizenConfig)
 register_architecture(VufizenConfig)
+register_architecture(LumedraConfig)

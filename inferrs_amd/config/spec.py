@@ -90,6 +90,11 @@ class AttentionSpec:
     mask_chunk: Optional[int] = None       # a query sees the keys of its own chunk of this many positions only (chunks counted from
                                            # position 0 of the sequence), up to itself; the cache keeps every position
     gate_per_head: bool = False            # with `gate`: one gate value a head ("g_proj.weight" is [n_heads, hidden])
+    keep_first: int = 0                    # with a window: a query sees the first so many positions besides, and the cache keeps them
+    softcap: Optional[float] = None        # a scaled score becomes softcap * tanh(score / softcap) ahead of the softmax
+    v_mix: Optional[str] = None            # "first": this layer's values of a step's tokens are left for later layers; "mix": values
+                                           # become (1 - l) v + l v_first before they are cached, l one learned number a layer.
+                                           # (the tensor "v_mix", of shape [])
     qk_unit_norm: bool = False             # q and k are brought to unit root mean square a head, without a weight (`qk_norm` gives
                                            # size and eps, no tensor is loaded).  A turn by position keeps a head's sum of
                                            # squares, so the norm ahead of the turn and behind it are the same number
@@ -143,6 +148,20 @@ class RetentionSpec:
     decay: Tuple[float, ...]
     norm_eps: float
     kind: str = "retention"
+
+
+@dataclass(frozen=True)
+class LightningSpec:
+    """Lightning attention: the fading sum of retention over activated rows, S <- decay_h S + k v^T, o = S^T q with q, k and
+    v each silu of its projection and no other scale.  The heads side by side are RMS-normed together (`norm_eps`, tensor
+    "norm" [n_heads * v_dim]), gated by sigmoid(W_g h) and go through W_o.  No biases."""
+    hidden: int
+    n_heads: int
+    head_dim: int
+    v_dim: int
+    decay: Tuple[float, ...]
+    norm_eps: float
+    kind: str = "lightning"
 
 
 @dataclass(frozen=True)
@@ -290,7 +309,8 @@ class RoutedExpertsSpec:
     the chosen experts (tensors under "shared."), its output added; `shared_gate`: times sigmoid(W_sg h), one number a
     token (tensor "shared.sg" [1, hidden], formed like a router's logit, in 32-bit).  `weight_on_input`: a chosen expert
     runs on weight * h and its output is added as it is (instead of weight * expert(h)).  `activation` "silu": an expert is
-    W_down (silu(W_gate h) * (W_up h)), without limits."""
+    W_down (silu(W_gate h) * (W_up h)), without limits.  `groups` (count, keep): the router's outputs form `count` equal groups
+    of neighbours; a group is worth the sum of its two largest scores, and the choice is among the `keep` best groups'."""
     hidden: int
     intermediate: int
     experts: int
@@ -307,6 +327,7 @@ class RoutedExpertsSpec:
     weight_on_input: bool = False
     shared_gate: bool = False
     activation: str = "clamped"
+    groups: Optional[Tuple[int, int]] = None
 
 
 @dataclass(frozen=True)
@@ -345,7 +366,8 @@ class TokenSideSpec:
 @dataclass(frozen=True)
 class ParallelSpec:
     """How a layer's sub-layers stand around a stream kept in 32-bit when both read ONE normed copy of it:
-    h = norm(x); x <- x + mixer(h) + ffn(h).  `side`: a `TokenSideSpec` whose row enters behind the sum."""
+    h = norm(x); x <- x + mixer(h) + ffn(h); or, with two norms in the layer, a normed copy each: x <- x + mixer(norm(x)) +
+    ffn(norm'(x)).  `side`: a `TokenSideSpec` whose row enters behind the sum."""
     side: Any = None
 
 
@@ -383,8 +405,8 @@ class LayerSpec:
     "streams" is pre-norm around several residual streams (`residual`: a `StreamsSpec`) and takes a
     layer without a feed-forward (`ffn` None, one norm); "post_norm" norms the stream after every sum (`residual`: a
     `PostNormSpec`; norms in the order behind the mixer, behind the feed-forward; one norm for a layer without one);
-    "parallel" has ONE norm, whose output both sub-layers read, and adds their outputs together (`residual`: a
-    `ParallelSpec`); "gated_branch" norms what a sub-layer gives, behind an optional gate (`residual`: a `GatedBranchSpec`;
+    "parallel" has ONE norm, whose output both sub-layers read, or one a sub-layer (mixer first), of the same rows, and adds
+    their outputs together (`residual`: a `ParallelSpec`); "gated_branch" norms what a sub-layer gives, behind an optional gate (`residual`: a `GatedBranchSpec`;
     norms in the order of the sub-layers).  `norms[i]` loads its weight from `norm_names[i]` (a norm with more tensors finds the others under
     that name plus a suffix of its spec's)."""
     mixer: Any

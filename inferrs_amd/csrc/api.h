@@ -44,11 +44,13 @@ int ia_qk_rope_kv(void* q_out, void* k_cache, void* v_cache, const void* qkv,
                   hipStream_t stream);
 
 // The same on rows of any layout (`ld_` elements a row: queries from q_off, keys from k_off, values of width dv from v_off; k_off < 0:
-// no keys or values, the layer reads another layer's cache)
+// no keys or values, the layer reads another layer's cache).  v_with: null, or another layer's values of the step's tokens
+// (value heads side by side, rows vw_ld apart): (1 - v_mix) v + v_mix v_with is what is cached
 int ia_qk_rope_kv_strided(void* q_out, void* k_cache, void* v_cache, const void* proj, const float* q_norm_w,
                           const float* k_norm_w, const float* cos_t, const float* sin_t, const int* slots, int n,
                           int ld_, int q_off, int k_off, int v_off, int nq, int nkv, int d, int dv, int rot,
-                          int interleaved, int page_size, float eps, int add_one, int dtype, hipStream_t stream);
+                          int interleaved, int page_size, float eps, int add_one, const void* v_with,
+                          long long vw_ld, float v_mix, int dtype, hipStream_t stream);
 
 // d: the keys' width, dv: the values' (v_cache [pages, nkv, dv, page_size], out [n, nq, dv])
 // sink: 1 adds exp(0) to the softmax's denominator (a key of score 0 that has no value); the same in the matrix-core kernels.
@@ -60,7 +62,7 @@ int ia_attention_generic(void* out, const void* q, const void* k_cache, const vo
                          const int* positions, const int* token_seq, const int* block_table,
                          int n, int max_pages, int nq, int nkv, int d, int dv, int page_size, int window,
                          float scale, int dtype, float* workspace, int max_kv_len, int sink, int mask_chunk,
-                         const float* sinks, hipStream_t stream);
+                         const float* sinks, int keep_first, float softcap, hipStream_t stream);
 long long ia_attention_generic_workspace(int n, int nq, int nkv, int d, int dv, int max_kv_len);
 
 int ia_gemm_tiled(void* out, const void* x, const void* w, int M, int N, int K, int in_dtype,
@@ -195,13 +197,15 @@ int ia_rglru_scan_chunked(void* out, float* state, float* work, const float* u, 
 // choice_bias: null, or [E] 32-bit values that count in the choice only (score + bias picks, the score weighs).  The plan
 // gives a pair whose choice is E or beyond (an output of the router that names no expert with weights) no place and no tile.
 int ia_route(int* sel, float* weight, const void* h, const void* router, int n, int W, int E, int top,
-             float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order,
-             int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, int dtype, hipStream_t stream);   // order: null, or the plan of ia_route_plan as well
+             float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int group_count,
+             int group_keep, int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, int dtype, hipStream_t stream);   // order: null, or the plan of ia_route_plan as well
+// (group_count > 1: the outputs form that many equal groups of neighbours, and only those of the group_keep groups with the
+// largest sums of two scores can be chosen)
 // the choice from logits that a product has left (32-bit rows of pitch ld from column off on: E experts, then the gates), up to
 // 16 tokens in one block, with the plan
 int ia_route_logits(int* sel, float* weight, const float* logits, long long ld, int off, int n, int E, int top, float scale,
-                    int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order, int* tile_expert,
-                    int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, hipStream_t stream);
+                    int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int group_count, int group_keep,
+                    int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, hipStream_t stream);
 int ia_route_plans(int n, int W, int rows, int dtype, const void* h, const void* router);    // 1: ia_route makes this step's plan itself
 int ia_route_tiles(int pairs, int E);
 int ia_route_plan(int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, const int* sel,
@@ -225,12 +229,13 @@ int ia_activation(void* x, long long n, int act, int dtype, hipStream_t stream);
 
 // A 32-bit residual stream whose sub-layers all read one normed copy (parallel.hip): x += y1 + y2 + sum_k [routed_w[k]] routed[k]
 // + y3_scale y3; x += rmsnorm(enter) * enter_w; h = norm(x) (a layer norm with weight and bias, or with center 0 an RMS norm):
-// every part optional, one kernel.  y_dtype: of y1, y2, y3, enter; h_dtype: of xr (the new x once more) and h.  rows: only these
+// every part optional, one kernel.  h2: the same rows through a second norm with a weight (and bias) of its own.  y_dtype: of y1, y2, y3, enter; h_dtype: of xr (the new x once more) and h.  rows: only these
 // rows through the norm, nothing added, the stream left alone.
 int ia_parallel_step(float* x, const void* y1, const void* y2, const void* y3, int y1_splits, int y2_splits, int y3_splits,
                      const float* y3_scale, const float* routed, const float* routed_w, int top, const void* enter,
                      const float* enter_w, float enter_eps, void* xr, const float* norm_w, const float* norm_b, float norm_eps,
-                     int center, void* h, const int* rows, int n, int W, int y_dtype, int h_dtype, hipStream_t stream);
+                     int center, void* h, const float* norm2_w, const float* norm2_b, void* h2, const int* rows, int n, int W,
+                     int y_dtype, int h_dtype, hipStream_t stream);
 // out[t][c] = act(g[t][c]) * e[t][e_off + c]; act: 1 SiLU, 2 GELU in its tanh form
 int ia_gate_rows(void* out, const void* g, const void* e, int rows, int cols, long long e_ld, int e_off, int act, int dtype,
                  hipStream_t stream);
@@ -264,7 +269,8 @@ int ia_exp_gates(float* log_a, float* b, float* floor_, float* state, long long 
 int ia_step_gates(float* log_a, float* b, const void* proj, long long p_ld, int dt_off, const float* dt_bias,
                   const float* a_log, int n, int H, int dtype, hipStream_t stream);
 // S <- a S + b k v^T, o = S^T q (+ skip v); `den` not null: one more column of S whose value is always 1.
-// log_a: [n][H] logarithms of the decays (a_per_token 1) or the decays themselves, [H] (a_per_token 0).
+// log_a: [n][H] logarithms of the decays (a_per_token 1) or the decays themselves, [H] (a_per_token 0).  act 1: q, k and v
+// through SiLU first (0: as they are).
 // chunk > 0: portions run in chunks of that many tokens side by side (workspace: ia_linear_scan_workspace floats; max_q_len:
 // an upper bound of a request's tokens); the results differ from the walk (chunk 0) by rounding.
 int ia_linear_scan(float* out, float* den, float* state, long long row_floats, long long s_off,
@@ -273,7 +279,7 @@ int ia_linear_scan(float* out, float* den, float* state, long long row_floats, l
                    const void* v, long long v_ld, int v_off,
                    const float* log_a, int a_per_token, const float* b, const float* skip,
                    const int* cu_tokens, const int* state_slots, int n_seqs, int H, int dim, int vdim,
-                   float q_scale, float k_scale, int chunk, int max_q_len, float* workspace, int dtype,
+                   float q_scale, float k_scale, int act, int chunk, int max_q_len, float* workspace, int dtype,
                    hipStream_t stream);
 long long ia_linear_scan_workspace(int n_seqs, int max_q_len, int chunk, int H, int dim, int vdim, int normaliser);
 // 1 (the default): what a chunk's start contributes is formed on the matrix cores in true 32-bit (keys up to 128, chunks up
@@ -319,7 +325,8 @@ int ia_attention_mfma(void* out, float* workspace, const void* q, const void* k_
                       const int* positions, int n, int seq_begin, int n_seqs, int token_begin,
                       int n_tokens, int max_q_len, int max_kv_len, int max_pages,
                       int nq, int nkv, int d, int page_size, int window, float scale,
-                      int splits, int chunk, int sink, int mask_chunk, const float* sinks, hipStream_t stream);
+                      int splits, int chunk, int sink, int mask_chunk, const float* sinks, int keep_first, float softcap,
+                      hipStream_t stream);
 // Decode steps (one token a request, head sizes in steps of 64): per-head norm, rotation, cache write, attention
 // and the merge of the key splits in one kernel.  `workspace` holds ia_attention_decode_workspace() floats;
 // `counters` holds at least ia_attention_decode_counters() 32-bit words that are zero before the call and zero

@@ -43,6 +43,24 @@ __device__ __forceinline__ float4 ag_load4(const bf16_t* p) {
                        bf16_bits_to_f32((uint16_t)v.y), bf16_bits_to_f32((uint16_t)(v.y >> 16)));
 }
 
+// Which keys a position sees and which tiles of them are walked: those below `keep` and those from `lo` on (keep < lo; keep
+// 0: no first ones, or nothing between them and the rest is hidden).  The tiles hole_lo .. hole_hi - 1 hold none of them.
+struct AgWalk {
+    int lo, keep, hole_lo, hole_hi;
+    __device__ __forceinline__ int from(int tile) const { return tile >= hole_lo && tile < hole_hi ? hole_hi : tile; }
+    __device__ __forceinline__ int tile0() const { return from(0); }
+    __device__ __forceinline__ bool skips(int seg) const { return seg * AG_SEG_TILES >= hole_lo && (seg + 1) * AG_SEG_TILES <= hole_hi; }
+};
+__device__ __forceinline__ AgWalk ag_walk(int pos, int window, int mask_chunk, int keep_first) {
+    AgWalk w;
+    w.lo = ia_key_floor(pos, window, mask_chunk);
+    w.keep = keep_first;
+    if (w.keep >= w.lo) { w.lo = 0; w.keep = 0; }
+    w.hole_lo = (w.keep + AG_TILE - 1) / AG_TILE;
+    w.hole_hi = w.lo / AG_TILE;
+    return w;
+}
+
 // Totals (big_m, big_l, big_o) take in a segment (m, l, o): the one place where this is written down.
 __device__ __forceinline__ void ag_merge_scales(float big_m, float m, float& m_out, float& a, float& b) {
     m_out = fmaxf(big_m, m);
@@ -68,7 +86,9 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
     int segs,
     int sink,                            // 1: the softmax's denominator holds one more term, exp(0): a key of score 0 without a value
     int mask_chunk,                      // > 0: a query sees the keys of its own chunk of this many positions only
-    const float* __restrict__ sinks) {   // with sink: null, or [nq] values s_h a query head; the term is exp(s_h), not scaled
+    const float* __restrict__ sinks,     // with sink: null, or [nq] values s_h a query head; the term is exp(s_h), not scaled
+    int keep_first,                      // the first so many positions are seen beside the window or chunk
+    float softcap) {                     // > 0: a score becomes softcap * tanh(score / softcap)
     __shared__ __attribute__((aligned(16))) float stage[AG_TILE * AG_PITCH];     // keys: [key][dim]; values: [dim][key]
     __shared__ __attribute__((aligned(16))) float sp[HEADS][AG_TILE];
     extern __shared__ __attribute__((aligned(16))) float ag_rows[];       // queries, a segment's outputs, the totals: [HEADS][dpad] each
@@ -84,7 +104,9 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
     const int heads = kvh * g + g - h0 < HEADS ? kvh * g + g - h0 : HEADS;
     const int pos = positions[tok];
     const int* bt = block_table + (size_t)token_seq[tok] * max_pages;
-    const int lo = ia_key_floor(pos, window, mask_chunk);
+    const AgWalk wk = ag_walk(pos, window, mask_chunk, keep_first);
+    const int lo = wk.lo, keep = wk.keep;
+    auto seen = [&](int key) { return key <= pos && (key >= lo || key < keep); };
     const int chunks = (d + AG_CHUNK - 1) / AG_CHUNK;                  // of a key's dimensions
     const int vchunks = (dv + AG_CHUNK - 1) / AG_CHUNK;                // of a value's
     const int dpad = (chunks > vchunks ? chunks : vchunks) * AG_CHUNK;
@@ -97,8 +119,8 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
         for (int e = lane; e < dpad; e += IA_WAVE)
             sq[h * dpad + e] = (h < heads && e < d) ? ld(q + ((size_t)tok * nq + h0 + h) * d + e) : 0.f;
 
-    const int seg_first = lo / AG_SEGMENT, seg_last = pos / AG_SEGMENT;
-    if (only_seg >= 0 && (only_seg < seg_first || only_seg > seg_last)) return;       // (the whole wave)
+    const int seg_first = wk.tile0() / AG_SEG_TILES, seg_last = pos / AG_SEGMENT;
+    if (only_seg >= 0 && (only_seg < seg_first || only_seg > seg_last || wk.skips(only_seg))) return;       // (the whole wave)
     float big_m[HEADS], big_l[HEADS];
 #pragma unroll
     for (int h = 0; h < HEADS; ++h) { big_m[h] = -INFINITY; big_l[h] = 0.f; }
@@ -106,13 +128,14 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
         for (int h = 0; h < HEADS; ++h)
             for (int e = lane; e < dpad; e += IA_WAVE) st_[h * dpad + e] = 0.f;
     for (int seg = only_seg >= 0 ? only_seg : seg_first; seg <= (only_seg >= 0 ? only_seg : seg_last); ++seg) {
+    if (wk.skips(seg)) continue;
     // the segment's outputs so far: lane e owns dimensions e, e + 64, ... of every head (nobody else touches them)
     for (int h = 0; h < HEADS; ++h)
         for (int e = lane; e < dpad; e += IA_WAVE) so[h * dpad + e] = 0.f;
     float m[HEADS], l[HEADS];
 #pragma unroll
     for (int h = 0; h < HEADS; ++h) { m[h] = -INFINITY; l[h] = 0.f; }
-    const int tile_first = seg * AG_SEG_TILES > lo / AG_TILE ? seg * AG_SEG_TILES : lo / AG_TILE;
+    const int tile_first = wk.from(seg * AG_SEG_TILES);
     const int tile_last = seg * AG_SEG_TILES + AG_SEG_TILES - 1 < pos / AG_TILE ? seg * AG_SEG_TILES + AG_SEG_TILES - 1 : pos / AG_TILE;
 
     // ---- the pieces of a tile's work (the same arithmetic in the same order whoever stages the operands) -----------
@@ -137,7 +160,9 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
     auto softmax = [&](bool valid) {
 #pragma unroll
         for (int h = 0; h < HEADS; ++h) {
-            const float sc = valid ? s[h] * scale : -INFINITY;
+            float sc = s[h] * scale;
+            if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+            sc = valid ? sc : -INFINITY;
             const float m_new = fmaxf(m[h], wave_max(sc));
             const float p = valid ? expf(sc - m_new) : 0.f;
             alpha[h] = expf(m[h] - m_new);
@@ -170,7 +195,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
     // key j's page of a tile, in lane j - j0: asked for once a tile, handed round
     auto tile_pages = [&](int tile) {
         const int j = tile * AG_TILE + lane;
-        return (j >= lo && j <= pos) ? bt[j / page_size] : 0;
+        return seen(j) ? bt[j / page_size] : 0;
     };
 
     if constexpr (VEC && AHEAD) {
@@ -196,7 +221,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                     const int key = j0 + r;
                     const int page = __shfl(pages, r);
                     held[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-                    if (key >= lo && key <= pos && e < d)
+                    if (seen(key) && e < d)
                         held[i] = ag_load4(k_cache + (((size_t)page * nkv + kvh) * page_size + key % page_size) * d + e);
                 }
             } else {
@@ -204,10 +229,10 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                 const int k4 = (lane & 15) * 4;
                 const int key = j0 + k4;
                 const int off = key % page_size;
-                const bool any = key + 3 >= lo && key <= pos;
+                const bool any = (key + 3 >= lo && key <= pos) || key < keep;
                 // the page of the four keys, from a lane whose key is in the range (a page that a window has passed is
                 // not in the table any more; the keys of these four that are in the range share their page)
-                const int first_in = key >= lo ? k4 : (lo - j0 < AG_TILE ? lo - j0 : k4);
+                const int first_in = key >= lo || key < keep ? k4 : (lo - j0 < AG_TILE ? lo - j0 : k4);
                 const int page = __shfl(pages, first_in);
 #pragma unroll
                 for (int i = 0; i < LOADS; ++i) {
@@ -226,8 +251,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
             } else {
                 const int k4 = (lane & 15) * 4;
                 const int key = tile * AG_TILE + k4;
-                const bool in0 = key >= lo && key <= pos, in1 = key + 1 >= lo && key + 1 <= pos;
-                const bool in2 = key + 2 >= lo && key + 2 <= pos, in3 = key + 3 >= lo && key + 3 <= pos;
+                const bool in0 = seen(key), in1 = seen(key + 1), in2 = seen(key + 2), in3 = seen(key + 3);
 #pragma unroll
                 for (int i = 0; i < LOADS; ++i) {
                     float4 v = held[i];
@@ -241,10 +265,11 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
         };
         int pages = tile_pages(tile_first);
         if (tile_first <= tile_last) ask(tile_first, 0, pages);
-        for (int tile = tile_first; tile <= tile_last; ++tile) {
+        for (int tile = tile_first, next; tile <= tile_last; tile = next) {
+            next = wk.from(tile + 1);
             const int j = tile * AG_TILE + lane;
-            const bool valid = j >= lo && j <= pos;
-            const int pages_next = tile < tile_last ? tile_pages(tile + 1) : 0;
+            const bool valid = seen(j);
+            const int pages_next = next <= tile_last ? tile_pages(next) : 0;
 #pragma unroll
             for (int h = 0; h < HEADS; ++h) s[h] = 0.f;
             for (int step = 0; step < steps; ++step) {
@@ -252,7 +277,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                 __syncthreads();                                      // the stage is free (and the probabilities are there)
                 put(tile, step);
                 if (step + 1 < steps) ask(tile, step + 1, pages);
-                else if (tile < tile_last) ask(tile + 1, 0, pages_next);
+                else if (next <= tile_last) ask(next, 0, pages_next);
                 __syncthreads();
                 if (step < chunks) scores(step);
                 else values(step - chunks);
@@ -260,10 +285,10 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
             pages = pages_next;
         }
     } else {
-    for (int tile = tile_first; tile <= tile_last; ++tile) {
+    for (int tile = tile_first; tile <= tile_last; tile = wk.from(tile + 1)) {
         const int j0 = tile * AG_TILE;
         const int j = j0 + lane;
-        const bool valid = j >= lo && j <= pos;
+        const bool valid = seen(j);
         const int my_page = tile_pages(tile);
 #pragma unroll
         for (int h = 0; h < HEADS; ++h) s[h] = 0.f;
@@ -279,7 +304,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                     const int key = j0 + r;
                     const int page = __shfl(my_page, r);
                     v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-                    if (key >= lo && key <= pos && e < d)
+                    if (seen(key) && e < d)
                         v[i] = ag_load4(k_cache + (((size_t)page * nkv + kvh) * page_size + key % page_size) * d + e);
                 }
 #pragma unroll
@@ -290,7 +315,7 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                     const int key = j0 + r, e = c * AG_CHUNK + lane;
                     float v = 0.f;
                     const int page = __shfl(my_page, r);
-                    if (key >= lo && key <= pos && e < d)
+                    if (seen(key) && e < d)
                         v = ld(k_cache + (((size_t)page * nkv + kvh) * page_size + key % page_size) * d + e);
                     stage[r * AG_PITCH + lane] = v;
                 }
@@ -306,10 +331,10 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                 const int k4 = (lane & 15) * 4;
                 const int key = j0 + k4;
                 const int off = key % page_size;                      // (four keys never straddle a page)
-                const bool any = key + 3 >= lo && key <= pos;
+                const bool any = (key + 3 >= lo && key <= pos) || key < keep;
                 // the page of the four keys, from a lane whose key is in the range (a page that a window has passed is
                 // not in the table any more; the keys of these four that are in the range share their page)
-                const int first_in = key >= lo ? k4 : (lo - j0 < AG_TILE ? lo - j0 : k4);
+                const int first_in = key >= lo || key < keep ? k4 : (lo - j0 < AG_TILE ? lo - j0 : k4);
                 const int page = __shfl(my_page, first_in);
                 float4 v[AG_CHUNK / 4];
 #pragma unroll
@@ -318,10 +343,10 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
                     v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
                     if (any && e < dv) {
                         v[i] = ag_load4(v_cache + (((size_t)page * nkv + kvh) * dv + e) * page_size + off);
-                        v[i].x = (key >= lo && key <= pos) ? v[i].x : 0.f;
-                        v[i].y = (key + 1 >= lo && key + 1 <= pos) ? v[i].y : 0.f;
-                        v[i].z = (key + 2 >= lo && key + 2 <= pos) ? v[i].z : 0.f;
-                        v[i].w = (key + 3 >= lo && key + 3 <= pos) ? v[i].w : 0.f;
+                        v[i].x = seen(key) ? v[i].x : 0.f;
+                        v[i].y = seen(key + 1) ? v[i].y : 0.f;
+                        v[i].z = seen(key + 2) ? v[i].z : 0.f;
+                        v[i].w = seen(key + 3) ? v[i].w : 0.f;
                     }
                 }
 #pragma unroll
@@ -374,18 +399,19 @@ __global__ __launch_bounds__(IA_WAVE) void attn_generic_kernel(
 template <typename T>
 __global__ __launch_bounds__(IA_WAVE) void attn_generic_merge_kernel(
     T* __restrict__ out, const float* __restrict__ partial, const int* __restrict__ positions, int nq, int d, int dpad,
-    int window, int segs, int sink, int mask_chunk, const float* __restrict__ sinks) {
+    int window, int segs, int sink, int mask_chunk, const float* __restrict__ sinks, int keep_first) {
     const int lane = threadIdx.x;
     const int tok = blockIdx.x / nq, h = blockIdx.x - tok * nq;
     const int pos = positions[tok];
-    const int lo = ia_key_floor(pos, window, mask_chunk);
+    const AgWalk wk = ag_walk(pos, window, mask_chunk, keep_first);
     float big_m = -INFINITY, big_l = 0.f;
     float big_o[AG_MAX_HEAD_DIM / IA_WAVE];
 #pragma unroll
     for (int t = 0; t < AG_MAX_HEAD_DIM / IA_WAVE; ++t) big_o[t] = 0.f;
     // (a position beyond the caller's bound has segments that nobody wrote: they are left out rather than read)
     const int seg_last = pos / AG_SEGMENT < segs - 1 ? pos / AG_SEGMENT : segs - 1;
-    for (int seg = lo / AG_SEGMENT; seg <= seg_last; ++seg) {
+    for (int seg = wk.tile0() / AG_SEG_TILES; seg <= seg_last; ++seg) {
+        if (wk.skips(seg)) continue;
         const float* row = partial + (((size_t)tok * nq + h) * segs + seg) * (dpad + 2);
         float m_out, a, b;
         ag_merge_scales(big_m, row[dpad], m_out, a, b);
@@ -423,8 +449,10 @@ extern "C" int ia_attention_generic(void* out, const void* q, const void* k_cach
                                     const int* positions, const int* token_seq, const int* block_table,
                                     int n, int max_pages, int nq, int nkv, int d, int dv, int page_size,
                                     int window, float scale, int dtype, float* workspace, int max_kv_len,
-                                    int sink, int mask_chunk, const float* sinks, hipStream_t stream) {
+                                    int sink, int mask_chunk, const float* sinks, int keep_first, float softcap,
+                                    hipStream_t stream) {
     IA_CHECK(mask_chunk >= 0 && (sinks == nullptr || sink), "attention: mask_chunk %d must be >= 0 (0 = none), and sink values go with a sink", mask_chunk);
+    IA_CHECK(keep_first >= 0 && softcap >= 0.f, "attention: keep_first %d and softcap %g must be >= 0 (0 = none)", keep_first, (double)softcap);
     IA_CHECK(n >= 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention: bad head counts nq=%d nkv=%d (n=%d)", nq, nkv, n);
     IA_CHECK(d > 0 && d <= AG_MAX_HEAD_DIM, "attention: head_dim %d is outside 1..%d", d, AG_MAX_HEAD_DIM);
     IA_CHECK(dv > 0 && dv <= AG_MAX_HEAD_DIM, "attention: the values' width %d is outside 1..%d", dv, AG_MAX_HEAD_DIM);
@@ -448,7 +476,7 @@ extern "C" int ia_attention_generic(void* out, const void* q, const void* k_cach
     const bool vec = d % 4 == 0 && dv % 4 == 0 && page_size % 4 == 0 &&
                      (((uintptr_t)k_cache | (uintptr_t)v_cache) % (4 * elem)) == 0;
 #define AG_ARGS(T) (T*)out, (const T*)q, (const T*)k_cache, (const T*)v_cache, positions, token_seq, block_table, max_pages, nq, nkv, \
-        d, dv, page_size, window, scale, workspace, segs, sink, mask_chunk, sinks
+        d, dv, page_size, window, scale, workspace, segs, sink, mask_chunk, sinks, keep_first, softcap
     // (a wave a segment, steps of few tokens: the operands are asked for a step ahead)
 #define AG_LAUNCH(T, V, H) do { \
         if (V && workspace != nullptr) attn_generic_kernel<T, V, H, true><<<grid, IA_WAVE, rows_bytes, stream>>>(AG_ARGS(T)); \
@@ -465,9 +493,9 @@ extern "C" int ia_attention_generic(void* out, const void* q, const void* k_cach
     IA_LAUNCH_CHECK("attention_generic");
     if (workspace != nullptr) {
         if (dtype == IA_F32)
-            attn_generic_merge_kernel<float><<<(unsigned)n * nq, IA_WAVE, 0, stream>>>((float*)out, workspace, positions, nq, dv, dpad, window, segs, sink, mask_chunk, sinks);
+            attn_generic_merge_kernel<float><<<(unsigned)n * nq, IA_WAVE, 0, stream>>>((float*)out, workspace, positions, nq, dv, dpad, window, segs, sink, mask_chunk, sinks, keep_first);
         else
-            attn_generic_merge_kernel<bf16_t><<<(unsigned)n * nq, IA_WAVE, 0, stream>>>((bf16_t*)out, workspace, positions, nq, dv, dpad, window, segs, sink, mask_chunk, sinks);
+            attn_generic_merge_kernel<bf16_t><<<(unsigned)n * nq, IA_WAVE, 0, stream>>>((bf16_t*)out, workspace, positions, nq, dv, dpad, window, segs, sink, mask_chunk, sinks, keep_first);
         IA_LAUNCH_CHECK("attention_generic_merge");
     }
     return 0;

@@ -85,7 +85,19 @@ struct AttnParams {
     int sink;                   // 1: the softmax's denominator holds one more term, 2^(0 - m): a key of score 0 without a value
     const float* sinks;         // with sink: null, or [nq] values s_h a query head (natural logarithm, not scaled): the term is 2^(s_h log2 e - m)
     int mask_chunk;             // > 0: a query sees the keys of its own chunk of this many positions only, up to itself
+    int keep_first;             // > 0: it sees the first so many positions besides (forms 1 and 2)
+    float cap_in;               // form 2: a raw score s stands for tanh(s * scale / cap); this is 2 log2(e) scale / cap, and scale_log2 is cap * log2(e)
 };
+
+// What the kernels of single waves and of tiles are compiled for beside a window, a chunk and a sink: nothing (0), first
+// positions that every query sees (1), these and capped scores (2).
+enum { FORM_PLAIN = 0, FORM_KEEP = 1, FORM_CAP = 2 };
+
+// tanh from the exponential of twice its argument: `x` is 2 log2(e) times it.  (Within 2^-22 of the value in absolute terms;
+// at both ends the exponential is 0 or infinite and the value -1 or 1.)
+__device__ __forceinline__ float tanh_exp2(float x) {
+    return __builtin_fmaf(-2.0f, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x) + 1.0f), 1.0f);
+}
 
 __device__ __forceinline__ uint4 zero4() { return make_uint4(0, 0, 0, 0); }
 
@@ -95,7 +107,7 @@ __device__ __forceinline__ float sink_term(const float* sinks, int head, float m
 }
 
 // One column block (16 * NB columns) of one request and key/value head, over one split of the keys.
-template <int NB>
+template <int NB, int FORM>
 __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, int kvh, int split, int seq) {
     const int lane = threadIdx.x;
     const int r = lane & 15, G = lane >> 4;
@@ -149,10 +161,20 @@ __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, i
     const int last_floor = ia_key_floor(pmax, p.window, p.mask_chunk);     // first key that the last column sees
     int lo = window_floor;
     int hi = pmax + 1;
+    // The first positions that every query sees are a range of steps of their own, [pre_lo, pre_hi), ahead of the rest;
+    // where no whole step lies between the two, the walk starts at 0.
+    const int keep = FORM != FORM_PLAIN ? p.keep_first : 0;
+    int pre_lo = 0, pre_hi = 0;
+    if (FORM != FORM_PLAIN && keep > 0) {
+        if (keep >= (window_floor & ~31)) lo = 0;
+        else pre_hi = (keep + 31) & ~31;
+    }
     if (p.splits > 1) {
         const int c_lo = split * p.chunk, c_hi = c_lo + p.chunk;
         lo = lo > c_lo ? lo : c_lo;
         hi = hi < c_hi ? hi : c_hi;
+        pre_lo = c_lo;
+        pre_hi = pre_hi < c_hi ? pre_hi : c_hi;
     }
     lo &= ~31;
 
@@ -243,13 +265,14 @@ __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, i
             // names some other page, which holds anything at all).  Their scores are masked below; their values
             // are zeroed here, for the same reason as the slots beyond the length.
             const int first_good = window_floor - (k0 + 8 * G);     // keys below this index are outside every window
+            const int kept = keep - (k0 + 8 * G);                   // (those below this one are first positions: seen)
             if (first_good > 0) {
 #pragma unroll
                 for (int db = 0; db < DBV; ++db) {
                     uint32_t w[4] = {op.v[db].x, op.v[db].y, op.v[db].z, op.v[db].w};
 #pragma unroll
                     for (int j = 0; j < 8; ++j)
-                        if (j < first_good) w[j >> 1] &= (j & 1) ? 0x0000ffffu : 0xffff0000u;
+                        if (j < first_good && (FORM == FORM_PLAIN || j >= kept)) w[j >> 1] &= (j & 1) ? 0x0000ffffu : 0xffff0000u;
                     op.v[db] = make_uint4(w[0], w[1], w[2], w[3]);
                 }
             }
@@ -271,14 +294,14 @@ __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, i
 #pragma unroll
             for (int t = 0; t < 2; ++t)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) sc[4 * t + i] = s[t][i];
+                for (int i = 0; i < 4; ++i) sc[4 * t + i] = FORM == FORM_CAP ? tanh_exp2(s[t][i] * p.cap_in) : s[t][i];
             if (edge) {
                 const int kbase_idx = k0 + 8 * G;
                 const int floor_key = ia_key_floor(pos[nb], p.window, p.mask_chunk);
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const int key = kbase_idx + j;
-                    if (key > pos[nb] || key < floor_key) sc[j] = -INFINITY;
+                    if (key > pos[nb] || (key < floor_key && (FORM == FORM_PLAIN || key >= keep))) sc[j] = -INFINITY;
                 }
             }
             float mx = fmaxf(fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3])), fmaxf(fmaxf(sc[4], sc[5]), fmaxf(sc[6], sc[7])));
@@ -335,12 +358,30 @@ __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, i
     //   v_permlane swaps instead of shared memory, late and early column blocks as separate waves
     //   instead of one after the other in a wave: within 1 % each.
     // - Addresses without a division in the step (above): 1 % at 2,048 tokens.
-    Place at = {lo / p.page, lo % p.page};
-    for (int k0 = lo; k0 < hi; k0 += 32) {
-        Operands op;
-        load_step(op, k0, at);
-        compute_step(op, k0);
-        advance(at, 32);
+    if constexpr (FORM == FORM_PLAIN) {
+        Place at = {lo / p.page, lo % p.page};
+        for (int k0 = lo; k0 < hi; k0 += 32) {
+            Operands op;
+            load_step(op, k0, at);
+            compute_step(op, k0);
+            advance(at, 32);
+        }
+    } else {
+        const bool two = pre_lo < pre_hi;               // (pre_hi <= hi: the first range lies below every window)
+        int k0 = two ? pre_lo : lo;
+        Place at = {k0 / p.page, k0 % p.page};
+        while (k0 < hi) {
+            Operands op;
+            load_step(op, k0, at);
+            compute_step(op, k0);
+            k0 += 32;
+            advance(at, 32);
+            if (two && k0 == pre_hi) {
+                k0 = lo;
+                at.idx = lo / p.page;
+                at.off = lo % p.page;
+            }
+        }
     }
 
     // ---- results: lane (col, G) holds dims 16 db + 4 G + i of its column ---------------------
@@ -378,7 +419,7 @@ __device__ __forceinline__ void attn_column_block(const AttnParams& p, int cb, i
 // start: under a causal mask the late blocks walk many keys and the early ones few, and every
 // pair walks about the same number, so all waves end together.  It pays when the step's queries
 // span most of the context; a short portion late in a long context has equal blocks already.
-template <int NB>
+template <int NB, int FORM>
 __global__ __launch_bounds__(IA_WAVE) __attribute__((amdgpu_waves_per_eu(HDMAX <= 128 ? 2 : 1, HDMAX > 64 ? 2 : 8)))
 void attn_mfma_kernel(const AttnParams p) {
     const int kvh = blockIdx.y / p.splits, split = blockIdx.y - kvh * p.splits;
@@ -387,13 +428,13 @@ void attn_mfma_kernel(const AttnParams p) {
     const int n_blocks = (n_cols + 16 * NB - 1) / (16 * NB);
     if (!p.pair) {
         // heavy column blocks first
-        if ((int)blockIdx.x < n_blocks) attn_column_block<NB>(p, n_blocks - 1 - (int)blockIdx.x, kvh, split, seq);
+        if ((int)blockIdx.x < n_blocks) attn_column_block<NB, FORM>(p, n_blocks - 1 - (int)blockIdx.x, kvh, split, seq);
         return;
     }
     const int late = n_blocks - 1 - (int)blockIdx.x, early = (int)blockIdx.x;
     if (late < early) return;
-    attn_column_block<NB>(p, late, kvh, split, seq);
-    if (early != late) attn_column_block<NB>(p, early, kvh, split, seq);
+    attn_column_block<NB, FORM>(p, late, kvh, split, seq);
+    if (early != late) attn_column_block<NB, FORM>(p, early, kvh, split, seq);
 }
 
 // The maximum / the sum over the four lanes that hold a column's values (lanes l, l ^ 16, l ^ 32, l ^ 48), in all
@@ -987,7 +1028,7 @@ __device__ __forceinline__ void lds_load16(const char* from, uint32_t lds_at) {
 #define TILE_NBW 2
 // NBW_: column tiles of 16 a wave.  One instead of two halves a block's columns (64) and doubles the blocks: for steps
 // whose blocks of 128 columns would leave compute units without one (short prompts, few heads).
-template <bool ENABLED = TILE_FITS, int NBW_ = TILE_NBW>
+template <bool ENABLED = TILE_FITS, int NBW_ = TILE_NBW, int FORM = FORM_PLAIN>
 __global__ __launch_bounds__(TILE_GROUPS * TILE_WAVES * IA_WAVE) __attribute__((amdgpu_waves_per_eu(2, 2)))
 void attn_tile_kernel(const AttnParams p) {
     if constexpr (ENABLED) {
@@ -1031,12 +1072,27 @@ void attn_tile_kernel(const AttnParams p) {
         int lo = bfloor;
         lo &= ~(TILE_STAGE - 1);
         int hi = bpmax + 1;
+        // the first positions that every query sees: stages of their own ahead of the rest, or, where no whole stage lies
+        // between the two, a walk from 0
+        const int keep = FORM != FORM_PLAIN ? p.keep_first : 0;
+        int pre_lo = 0, pre_hi = 0;
+        if (FORM != FORM_PLAIN && keep > 0) {
+            if (keep >= lo) lo = 0;
+            else pre_hi = (keep + TILE_STAGE - 1) & ~(TILE_STAGE - 1);
+        }
         if (p.splits > 1) {             // this block's share of the keys (`chunk` is a multiple of a stage)
             const int c_lo = split * p.chunk, c_hi = c_lo + p.chunk;
             lo = lo > c_lo ? lo : c_lo;
             hi = hi < c_hi ? hi : c_hi;
+            pre_lo = c_lo;
+            pre_hi = pre_hi < c_hi ? pre_hi : c_hi;
         }
-        const int stages = hi > lo ? (hi - lo + TILE_STAGE - 1) / TILE_STAGE : 0;
+        const int pre_stages = FORM != FORM_PLAIN && pre_lo < pre_hi ? (pre_hi - pre_lo) / TILE_STAGE : 0;
+        const int stages = pre_stages + (hi > lo ? (hi - lo + TILE_STAGE - 1) / TILE_STAGE : 0);
+        auto stage_key = [&](int s) {   // the first key of stage s
+            if (FORM == FORM_PLAIN) return lo + s * TILE_STAGE;
+            return s < pre_stages ? pre_lo + s * TILE_STAGE : lo + (s - pre_stages) * TILE_STAGE;
+        };
 
         // this wave's columns (a wave without any still brings its share of the stages)
         const int col0 = bcol0 + wave * WAVE_COLS;
@@ -1092,7 +1148,7 @@ void attn_tile_kernel(const AttnParams p) {
             pages_reg = bt[idx < last_idx ? idx : last_idx];
         };
         auto pages_for = [&](int s, int& page, int& off) {
-            const int key0 = lo + s * TILE_STAGE + 16 * wave_s;
+            const int key0 = stage_key(s) + 16 * wave_s;
             const int k = key0 < kv_total ? key0 : (kv_total - 1) & ~15;
             const int idx = k / p.page;
             if (idx >= pages_base + IA_WAVE) pages_load(idx);
@@ -1124,11 +1180,12 @@ void attn_tile_kernel(const AttnParams p) {
         // So may the values of keys below the block's window, between the stage's start and the first key that any
         // of its columns sees: the window has passed them, and their pages may have been given back.
         auto zero_tail = [&](int s, char* buf) {
-            const int kb = lo + s * TILE_STAGE;
+            const int kb = stage_key(s);
             const int mine = kb + 16 * wave_s + 8 * v_half;          // the first of this lane's eight keys
             const int first_bad = kb + TILE_STAGE <= kv_total ? 8 : kv_total - mine;
             const int first_good = kb < bfloor ? bfloor - mine : 0;
             if (first_bad >= 8 && first_good <= 0) return;
+            const int kept = keep - mine;                            // (keys below this index are first positions: seen)
 #pragma unroll
             for (int c = 0; c < TILE_V_CHUNKS; ++c) {
                 uint4* at = (uint4*)(buf + TILE_K_BYTES + wave_s * (16 * HDV * 2) + c * 1024 + lane * 16);
@@ -1136,7 +1193,7 @@ void attn_tile_kernel(const AttnParams p) {
                 uint32_t w[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
                 for (int j = 0; j < 8; ++j)
-                    if (j >= first_bad || j < first_good) w[j >> 1] &= (j & 1) ? 0x0000ffffu : 0xffff0000u;
+                    if (j >= first_bad || (j < first_good && (FORM == FORM_PLAIN || j >= kept))) w[j >> 1] &= (j & 1) ? 0x0000ffffu : 0xffff0000u;
                 *at = make_uint4(w[0], w[1], w[2], w[3]);
             }
         };
@@ -1166,14 +1223,14 @@ void attn_tile_kernel(const AttnParams p) {
             // of a pass's 6,500, all at the same time (8,192 tokens 736 -> 655 us).
             const bool more = s + TILE_GROUPS < stages;
             if (more && kg == 0) issue(other, page_l, off_l);
-            const int kb = lo + s * TILE_STAGE;
+            const int kb = stage_key(s);
             // Steps of 32 keys.  A wave's operands are asked for a phase ahead of their use: the values of a
             // step before its softmax is worked out, the keys of the next step before this step's second
             // product, so that the shared memory's latency passes behind arithmetic.
             bool live[2];
 #pragma unroll
             for (int u = 0; u < 2; ++u)        // something of the step is visible to this wave's columns
-                live[u] = !(kb + 32 * u > pmax || kb + 32 * u + 31 < wlo);
+                live[u] = !(kb + 32 * u > pmax || (kb + 32 * u + 31 < wlo && (FORM == FORM_PLAIN || kb + 32 * u >= keep)));
             uint4 kop[2][KS];
             auto read_keys = [&](int u) {
 #pragma unroll
@@ -1204,14 +1261,14 @@ void attn_tile_kernel(const AttnParams p) {
 #pragma unroll
                 for (int t = 0; t < 2; ++t)
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) sc[4 * t + i] = sacc[t][i];
+                    for (int i = 0; i < 4; ++i) sc[4 * t + i] = FORM == FORM_CAP ? tanh_exp2(sacc[t][i] * p.cap_in) : sacc[t][i];
                 if constexpr (EDGE) {
                     const int kbase_idx = k0 + 8 * G;
                     const int floor_key = ia_key_floor(pos[nb], p.window, p.mask_chunk);
 #pragma unroll
                     for (int j = 0; j < 8; ++j) {
                         const int key = kbase_idx + j;
-                        if (key > pos[nb] || key < floor_key) sc[j] = -INFINITY;
+                        if (key > pos[nb] || (key < floor_key && (FORM == FORM_PLAIN || key >= keep))) sc[j] = -INFINITY;
                     }
                 }
                 // (the compiler's own maximum: written out as v_max3 instructions, which the compiler does not check
@@ -1327,7 +1384,7 @@ void attn_tile_kernel(const AttnParams p) {
         // A group's walk: its stages are kg, kg + 2, ...; both groups pass the same number of barriers.
         auto walk = [&](char* first, char* second) __attribute__((always_inline)) {
             if (kg < stages) {
-                const int key0 = lo + kg * TILE_STAGE + 16 * wave_s;
+                const int key0 = stage_key(kg) + 16 * wave_s;
                 pages_load((key0 < kv_total ? key0 : (kv_total - 1) & ~15) / p.page);
                 pages_for(kg, page_l, off_l);
                 issue(first, page_l, off_l);
@@ -1579,8 +1636,8 @@ static int attention_launch(void* out, float* workspace, const void* q, const vo
                             const int* positions, int n, int seq_begin, int n_seqs, int token_begin,
                             int n_tokens, int max_q_len, int max_kv_len, int max_pages,
                             int nq, int nkv, int d, int page_size, int window, float scale,
-                            int splits, int chunk, int sink, int mask_chunk, const float* sinks, const FusedArgs* fused,
-                            hipStream_t stream) {
+                            int splits, int chunk, int sink, int mask_chunk, const float* sinks, int keep_first, float softcap,
+                            const FusedArgs* fused, hipStream_t stream) {
     IA_CHECK(d == HD, "attention_mfma: built for head_dim %d, called with %d", HD, d);
     IA_CHECK(n >= 0 && n_seqs >= 0 && nq > 0 && nkv > 0 && nq % nkv == 0,
              "attention_mfma: bad sizes n=%d seqs=%d nq=%d nkv=%d", n, n_seqs, nq, nkv);
@@ -1616,6 +1673,13 @@ static int attention_launch(void* out, float* workspace, const void* q, const vo
     p.sink = sink ? 1 : 0;
     IA_CHECK(mask_chunk >= 0 && (sinks == nullptr || sink), "attention_mfma: mask_chunk %d must be >= 0 (0 = none), and sink values go with a sink", mask_chunk);
     p.sinks = sinks; p.mask_chunk = mask_chunk;
+    IA_CHECK(keep_first >= 0 && softcap >= 0.f, "attention_mfma: keep_first %d and softcap %g must be >= 0 (0 = none)", keep_first, (double)softcap);
+    p.keep_first = keep_first; p.cap_in = 0.f;
+    if (softcap > 0.f) {
+        p.cap_in = scale / softcap * (2.0f * 1.4426950408889634f);
+        p.scale_log2 = softcap * 1.4426950408889634f;
+    }
+    const int form = softcap > 0.f ? FORM_CAP : keep_first > 0 ? FORM_KEEP : FORM_PLAIN;
     const long long cols = (long long)max_q_len * g;
     // Columns a wave: 16 for decode, 32 for portions of prompts.  (64 keep every loaded key and
     // value in use for twice as many products but need the registers of a whole SIMD; with 32
@@ -1625,6 +1689,7 @@ static int attention_launch(void* out, float* workspace, const void* q, const vo
     const long long col_blocks = (cols + 16 * nb - 1) / (16 * nb);
     const dim3 grid((unsigned)(p.pair ? (col_blocks + 1) / 2 : col_blocks), nkv * splits, n_seqs);
     if (fused != nullptr) {
+        IA_CHECK(form == FORM_PLAIN, "attention_mfma: the fused form takes no kept first positions and no capped scores");
         IA_CHECK(HD % 64 == 0 && HDV == HD && max_q_len == 1, "attention_mfma: the fused form takes single tokens, head sizes in "
                  "steps of 64 and values as wide as keys (head size %d, %d tokens a request)", HD, max_q_len);
         p.qkv = (const bf16_t*)fused->qkv;
@@ -1665,12 +1730,25 @@ static int attention_launch(void* out, float* workspace, const void* q, const vo
         IA_CHECK(tiles <= 65535, "attention_mfma: %lld tiles of columns in a request (at most 65535)", tiles);
         const dim3 tgrid((unsigned)(nkv * splits * n_seqs), (unsigned)tiles, 1);
         p.pair = 0;
-        if (narrow) attn_tile_kernel<TILE_FITS, 1><<<tgrid, TILE_GROUPS * TILE_WAVES * IA_WAVE, 0, stream>>>(p);
-        else attn_tile_kernel<><<<tgrid, TILE_GROUPS * TILE_WAVES * IA_WAVE, 0, stream>>>(p);
-    } else if (nb == 1) {
-        attn_mfma_kernel<1><<<grid, IA_WAVE, 0, stream>>>(p);
+#define ATTN_TILE(FORM)                                                                                                        \
+        do {                                                                                                                   \
+            if (narrow) attn_tile_kernel<TILE_FITS, 1, FORM><<<tgrid, TILE_GROUPS * TILE_WAVES * IA_WAVE, 0, stream>>>(p);       \
+            else attn_tile_kernel<TILE_FITS, TILE_NBW, FORM><<<tgrid, TILE_GROUPS * TILE_WAVES * IA_WAVE, 0, stream>>>(p);       \
+        } while (0)
+        if (form == FORM_PLAIN) ATTN_TILE(FORM_PLAIN);
+        else if (form == FORM_KEEP) ATTN_TILE(FORM_KEEP);
+        else ATTN_TILE(FORM_CAP);
+#undef ATTN_TILE
     } else {
-        attn_mfma_kernel<2><<<grid, IA_WAVE, 0, stream>>>(p);
+#define ATTN_WAVES(FORM)                                                       \
+        do {                                                                   \
+            if (nb == 1) attn_mfma_kernel<1, FORM><<<grid, IA_WAVE, 0, stream>>>(p); \
+            else attn_mfma_kernel<2, FORM><<<grid, IA_WAVE, 0, stream>>>(p);   \
+        } while (0)
+        if (form == FORM_PLAIN) ATTN_WAVES(FORM_PLAIN);
+        else if (form == FORM_KEEP) ATTN_WAVES(FORM_KEEP);
+        else ATTN_WAVES(FORM_CAP);
+#undef ATTN_WAVES
     }
     IA_LAUNCH_CHECK("attention_mfma");
     if (splits > 1) {
@@ -1693,10 +1771,10 @@ extern "C" int ia_attention_mfma(void* out, float* workspace, const void* q, con
                                  int n_tokens, int max_q_len, int max_kv_len, int max_pages,
                                  int nq, int nkv, int d, int page_size, int window, float scale,
                                  int splits, int chunk, int sink, int mask_chunk, const float* sinks,
-                                 hipStream_t stream) {
+                                 int keep_first, float softcap, hipStream_t stream) {
     return attention_launch(out, workspace, q, k_cache, v_cache, block_table, cu_tokens, positions, n, seq_begin,
                             n_seqs, token_begin, n_tokens, max_q_len, max_kv_len, max_pages, nq, nkv, d, page_size,
-                            window, scale, splits, chunk, sink, mask_chunk, sinks, nullptr, stream);
+                            window, scale, splits, chunk, sink, mask_chunk, sinks, keep_first, softcap, nullptr, stream);
 }
 
 // Whether this head size has the fused decode form.
@@ -1723,5 +1801,5 @@ extern "C" int ia_attention_mfma_decode_fused(void* out, float* workspace, const
     const FusedArgs fused = {qkv, q_norm_w, k_norm_w, cos_t, sin_t, slots, eps, add_one, counters, n_counters};
     return attention_launch(out, workspace, nullptr, k_cache, v_cache, block_table, cu_tokens, positions, n, seq_begin,
                             n_seqs, token_begin, n_tokens, 1, max_kv_len, max_pages, nq, nkv, d, page_size,
-                            window, scale, splits, chunk, sink, 0, nullptr, &fused, stream);
+                            window, scale, splits, chunk, sink, 0, nullptr, 0, 0.f, &fused, stream);
 }

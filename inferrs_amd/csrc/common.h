@@ -59,7 +59,8 @@ __device__ __forceinline__ float gate_act(float g, int act) {
 // The first key that the query at `pos` sees (it sees every key from there up to itself).  window > 0: the last `window`
 // positions, itself included; mask_chunk > 0: the keys of its own chunk of `mask_chunk` positions, chunks counted from
 // position 0 of the sequence; both 0: every key.  The floor never falls as `pos` grows, which is what the kernels that
-// walk the keys of several queries together rest on.
+// walk the keys of several queries together rest on.  (First positions that every query sees besides, `keep_first`, are a
+// range of their own in those kernels.)
 __host__ __device__ __forceinline__ int ia_key_floor(int pos, int window, int mask_chunk) {
     int lo = window > 0 && pos - window + 1 > 0 ? pos - window + 1 : 0;
     if (mask_chunk > 0) {

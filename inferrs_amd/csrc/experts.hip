@@ -39,7 +39,8 @@ __device__ __forceinline__ void load8(const bf16_t* p, float (&v)[8]) {
 template <int Q>
 __device__ __forceinline__ void route_pick(int* __restrict__ sel, float* __restrict__ weight, const float* logits, int t, int lane, int E,
                                            int top, float scale, int score_fn, int renorm, const float* __restrict__ choice_bias,
-                                           int gates, float* __restrict__ gate_out, int* chosen = nullptr) {
+                                           int gates, float* __restrict__ gate_out, int group_count, int group_keep,
+                                           int* chosen = nullptr) {
     if (gates > 0) {
         E -= gates;
         for (int j = lane; j < gates; j += IA_WAVE) gate_out[(long long)t * gates + j] = 1.0f / (1.0f + expf(-logits[E + j]));
@@ -60,6 +61,46 @@ __device__ __forceinline__ void route_pick(int* __restrict__ sel, float* __restr
         for (int q = 0; q < Q; ++q) s += z[q] > -INFINITY ? expf(z[q] - zmax) : 0.f;
         denom = wave_sum(s);
     }
+    auto score = [&](float x) { return score_fn == IA_SCORE_SOFTMAX ? expf(x - zmax) / denom : 1.0f / (1.0f + expf(-x)); };
+    if (group_count > 1) {
+        // The outputs form `group_count` groups of neighbours; a group is worth the sum of its two largest scores (with the
+        // choice's bias), and only outputs of the `group_keep` best groups stay in the choice (of equal groups the lower).
+        const int size = E / group_count;
+        float worth[Q];     // group g lives in lane g % 64, register g / 64
+#pragma unroll
+        for (int q = 0; q < Q; ++q) {
+            const int g = q * IA_WAVE + lane;
+            float one = -INFINITY, two = -INFINITY;
+            for (int i = 0; g < group_count && i < size; ++i) {
+                const int e = g * size + i;
+                const float s = score(logits[e]) + (choice_bias != nullptr ? choice_bias[e] : 0.f);
+                if (s > one) { two = one; one = s; }
+                else if (s > two) two = s;
+            }
+            worth[q] = g < group_count ? one + (size > 1 ? two : 0.f) : -INFINITY;
+        }
+        int in = 0;         // bit q: the group in register q stays
+        for (int k = 0; k < group_keep; ++k) {
+            float best = -INFINITY;
+            int best_g = 0x7fffffff;
+#pragma unroll
+            for (int q = 0; q < Q; ++q)
+                if (!((in >> q) & 1) && worth[q] > best) { best = worth[q]; best_g = q * IA_WAVE + lane; }
+#pragma unroll
+            for (int o = IA_WAVE / 2; o > 0; o >>= 1) {
+                const float ob = __shfl_xor(best, o, IA_WAVE);
+                const int og = __shfl_xor(best_g, o, IA_WAVE);
+                if (ob > best || (ob == best && og < best_g)) { best = ob; best_g = og; }
+            }
+            if (best_g % IA_WAVE == lane) in |= 1 << (best_g / IA_WAVE);
+        }
+#pragma unroll
+        for (int q = 0; q < Q; ++q) {
+            const int e = q * IA_WAVE + lane, g = e < E ? e / size : 0;
+            const int kept = __shfl(in, g % IA_WAVE, IA_WAVE);
+            if (!((kept >> (g / IA_WAVE)) & 1)) z[q] = -INFINITY;
+        }
+    }
     float total = 0.f, mine = 0.f;
     int mine_e = 0;
     if (choice_bias != nullptr) {
@@ -69,8 +110,8 @@ __device__ __forceinline__ void route_pick(int* __restrict__ sel, float* __restr
 #pragma unroll
         for (int q = 0; q < Q; ++q) {
             const int e = q * IA_WAVE + lane;
-            sc[q] = e < E ? (score_fn == IA_SCORE_SOFTMAX ? expf(z[q] - zmax) / denom : 1.0f / (1.0f + expf(-z[q]))) : 0.f;
-            key[q] = e < E ? sc[q] + choice_bias[e] : -INFINITY;
+            sc[q] = e < E ? score(z[q]) : 0.f;
+            key[q] = e < E && z[q] > -INFINITY ? sc[q] + choice_bias[e] : -INFINITY;
         }
         for (int k = 0; k < top; ++k) {
             float best = -INFINITY, best_s = 0.f;
@@ -107,14 +148,14 @@ __device__ __forceinline__ void route_pick(int* __restrict__ sel, float* __restr
 #pragma unroll
         for (int q = 0; q < Q; ++q)
             if (best_e == q * IA_WAVE + lane) z[q] = -INFINITY;
-        const float s = score_fn == IA_SCORE_SOFTMAX ? expf(best - zmax) / denom : 1.0f / (1.0f + expf(-best));
+        const float s = score(best);
         total += s;
         if (lane == k) { mine = s; mine_e = best_e; }
     }
     if (lane < top) {
         sel[(long long)t * top + lane] = mine_e;
         if (chosen != nullptr) chosen[lane] = mine_e;
-        weight[(long long)t * top + lane] = (renorm ? mine / total : mine) * scale;
+        weight[(long long)t * top + lane] = (renorm ? mine / (total + 1e-20f) : mine) * scale;     // (scores that are all zero stay zero)
     }
 }
 
@@ -133,7 +174,7 @@ __global__ __launch_bounds__(64 * WAVES) void route_kernel(int* __restrict__ sel
                                                                     const T* __restrict__ h, const T* __restrict__ wr, int n,
                                                                     int W, int E, int top, float scale, int score_fn,
                                                                     int renorm, const float* __restrict__ choice_bias,
-                                                                    int gates, float* __restrict__ gate_out) {
+                                                                    int gates, float* __restrict__ gate_out, int group_count, int group_keep) {
     // E counts every row of the router's matrix: the last `gates` of them take no part in the choice; the sigmoid of
     // such a row's logit is handed out as it is (gate_out [n, gates]): a gate a token, formed like a router's logit.
     __shared__ float logits[IA_MAX_EXPERTS];
@@ -176,7 +217,7 @@ __global__ __launch_bounds__(64 * WAVES) void route_kernel(int* __restrict__ sel
     }
     __syncthreads();
     if (wave != 0) return;
-    route_pick<IA_MAX_EXPERTS / IA_WAVE>(sel, weight, logits, t, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out);
+    route_pick<IA_MAX_EXPERTS / IA_WAVE>(sel, weight, logits, t, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out, group_count, group_keep);
 }
 
 // The whole block.  `order` [pairs]: the pairs grouped by expert; tiles: expert, first place in `order`, rows; meta[0]: tiles.
@@ -243,7 +284,7 @@ __global__ __launch_bounds__(64 * IA_RM_WAVES) void route_mfma_kernel(int* __res
                                                                       const bf16_t* __restrict__ h, const bf16_t* __restrict__ wr, int n,
                                                                       int W, int E, int top, float scale, int score_fn, int renorm,
                                                                       const float* __restrict__ choice_bias, int gates,
-                                                                      float* __restrict__ gate_out, const RoutePlan plan) {
+                                                                      float* __restrict__ gate_out, int group_count, int group_keep, const RoutePlan plan) {
     extern __shared__ float rm_part[];             // [waves][tokens][16 NT]
     __shared__ float logits[IA_RM_TOKENS][16 * NT];
     __shared__ int chosen[IA_RM_TOKENS * IA_MAX_TOP];
@@ -282,7 +323,7 @@ __global__ __launch_bounds__(64 * IA_RM_WAVES) void route_mfma_kernel(int* __res
     }
     __syncthreads();
     if (t0 + wave < n)
-        route_pick<1>(sel, weight, logits[wave], t0 + wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out,
+        route_pick<1>(sel, weight, logits[wave], t0 + wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out, group_count, group_keep,
                       chosen + wave * top);
     if (plan.order == nullptr) return;             // (the same for all threads; the grid is one block otherwise)
     __syncthreads();
@@ -296,16 +337,16 @@ __global__ __launch_bounds__(64 * IA_RM_WAVES) void route_logits_kernel(int* __r
                                                                         const float* __restrict__ logits, long long ld, int n, int E,
                                                                         int top, float scale, int score_fn, int renorm,
                                                                         const float* __restrict__ choice_bias, int gates,
-                                                                        float* __restrict__ gate_out, const RoutePlan plan) {
+                                                                        float* __restrict__ gate_out, int group_count, int group_keep, const RoutePlan plan) {
     __shared__ int chosen[IA_RM_TOKENS * IA_MAX_TOP];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     if (wave < n) {
         if (E - gates <= IA_WAVE)
-            route_pick<1>(sel, weight, logits + wave * ld, wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out,
+            route_pick<1>(sel, weight, logits + wave * ld, wave, lane, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out, group_count, group_keep,
                           chosen + wave * top);
         else
             route_pick<IA_MAX_EXPERTS / IA_WAVE>(sel, weight, logits + wave * ld, wave, lane, E, top, scale, score_fn, renorm, choice_bias,
-                                                 gates, gate_out, chosen + wave * top);
+                                                 gates, gate_out, group_count, group_keep, chosen + wave * top);
     }
     __syncthreads();
     route_plan_block(plan, chosen, n * top);
@@ -459,16 +500,23 @@ extern "C" int ia_route_plans(int n, int W, int rows, int dtype, const void* h, 
     return n <= IA_RM_TOKENS && route_mfma_fits(W, rows, dtype, h, router) ? 1 : 0;
 }
 
+// group_count 0 or 1: no groups; else the outputs form that many equal groups of neighbours, of which the group_keep best (by
+// the sum of their two largest scores) stay in the choice.
+static bool route_groups_fit(int E, int top, int group_count, int group_keep) {
+    return group_count <= 1 || (E % group_count == 0 && group_keep >= 1 && group_keep <= group_count && top <= group_keep * (E / group_count));
+}
+
 // choice_bias: null, or [E] 32-bit values added to the scores for the choice only (the weights are the scores themselves)
 extern "C" int ia_route(int* sel, float* weight, const void* h, const void* router, int n, int W, int E, int top,
                         float scale, int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out,
-                        int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile,
-                        int dtype, hipStream_t stream) {
+                        int group_count, int group_keep, int* order, int* tile_expert, int* tile_first, int* tile_rows,
+                        int* meta, int plan_E, int tile, int dtype, hipStream_t stream) {
     // order: null, or the plan of `ia_route_plan` is made as well (ia_route_plans(...) says for which steps)
     // E: the router's outputs that can be chosen; the matrix holds `gates` more rows behind them (see the kernel)
     IA_CHECK(gates >= 0 && (gates == 0 || gate_out != nullptr), "route: %d gate rows need a place for their values", gates);
     IA_CHECK(n >= 0 && W > 0 && E >= 1 && E + gates <= IA_MAX_EXPERTS && top >= 1 && top <= E && top <= IA_MAX_TOP,
              "route: n=%d width=%d experts=%d and %d gate rows (up to %d) top=%d (up to %d)", n, W, E, gates, IA_MAX_EXPERTS, top, IA_MAX_TOP);
+    IA_CHECK(route_groups_fit(E, top, group_count, group_keep), "route: %d of %d groups of %d outputs, top %d", group_keep, group_count, E, top);
     E += gates;
     IA_CHECK(score_fn == IA_SCORE_SIGMOID || score_fn == IA_SCORE_SOFTMAX, "route: unknown score function %d", score_fn);
     IA_CHECK(order == nullptr || ia_route_plans(n, W, E, dtype, h, router), "route: this step's plan is made by a kernel of its own");
@@ -489,7 +537,7 @@ extern "C" int ia_route(int* sel, float* weight, const void* h, const void* rout
             asked = 1;                                                                                                  \
         }                                                                                                               \
         route_mfma_kernel<NT><<<blocks, 64 * IA_RM_WAVES, shm, stream>>>(sel, weight, (const bf16_t*)h, (const bf16_t*)router, n, W, E, top, \
-                                                                         scale, score_fn, renorm, choice_bias, gates, gate_out, plan); \
+                                                                         scale, score_fn, renorm, choice_bias, gates, gate_out, group_count, group_keep, plan); \
     } while (0)
         switch (nt) { case 1: IA_RM(1); break; case 2: IA_RM(2); break; case 3: IA_RM(3); break; default: IA_RM(4); break; }
 #undef IA_RM
@@ -497,7 +545,7 @@ extern "C" int ia_route(int* sel, float* weight, const void* h, const void* rout
         return 0;
     }
     const bool vec = W % 8 == 0 && tile_mfma_aligned(h) && tile_mfma_aligned(router);
-#define IA_ROUTE_SW(T, V, S, WV) route_kernel<T, V, S, WV><<<n, 64 * WV, 0, stream>>>(sel, weight, (const T*)h, (const T*)router, n, W, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out)
+#define IA_ROUTE_SW(T, V, S, WV) route_kernel<T, V, S, WV><<<n, 64 * WV, 0, stream>>>(sel, weight, (const T*)h, (const T*)router, n, W, E, top, scale, score_fn, renorm, choice_bias, gates, gate_out, group_count, group_keep)
 #define IA_ROUTE_S(T, V, S) IA_ROUTE_SW(T, V, S, IA_ROUTE_WAVES)
     // (up to 32 outputs: 8 a wave; up to 64: as many a wave as take them all in one walk over the row.  A step of few
     // tokens has few blocks, and a wave's walk is a chain of trips to the memory: sixteen waves a token then, each with
@@ -517,8 +565,10 @@ extern "C" int ia_route(int* sel, float* weight, const void* h, const void* rout
 }
 
 extern "C" int ia_route_logits(int* sel, float* weight, const float* logits, long long ld, int off, int n, int E, int top, float scale,
-                               int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int* order,
-                               int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E, int tile, hipStream_t stream) {
+                               int score_fn, int renorm, const float* choice_bias, int gates, float* gate_out, int group_count,
+                               int group_keep, int* order, int* tile_expert, int* tile_first, int* tile_rows, int* meta, int plan_E,
+                               int tile, hipStream_t stream) {
+    IA_CHECK(route_groups_fit(E, top, group_count, group_keep), "route_logits: %d of %d groups of %d outputs, top %d", group_keep, group_count, E, top);
     IA_CHECK(n >= 0 && n <= IA_RM_TOKENS && E >= 1 && gates >= 0 && E + gates <= IA_MAX_EXPERTS && top >= 1 && top <= E && top <= IA_MAX_TOP &&
              off >= 0 && off + E + gates <= ld && (gates == 0 || gate_out != nullptr) && order != nullptr,
              "route_logits: n=%d (up to %d) experts=%d and %d gates at %d of rows of %lld, top=%d", n, IA_RM_TOKENS, E, gates, off, ld, top);
@@ -528,7 +578,7 @@ extern "C" int ia_route_logits(int* sel, float* weight, const float* logits, lon
     plan.order = order; plan.tile_expert = tile_expert; plan.tile_first = tile_first; plan.tile_rows = tile_rows; plan.meta = meta;
     plan.E = plan_E; plan.tile = tile;
     route_logits_kernel<<<1, 64 * IA_RM_WAVES, 0, stream>>>(sel, weight, logits + off, ld, n, E + gates, top, scale, score_fn, renorm,
-                                                            choice_bias, gates, gate_out, plan);
+                                                            choice_bias, gates, gate_out, group_count, group_keep, plan);
     IA_LAUNCH_CHECK("route_logits");
     return 0;
 }

@@ -1,7 +1,7 @@
 // Mixers that carry a matrix of fixed size a head from token to token (linear attention in its recurrent form):
 //     S_t = a_t S_(t-1) + b_t k_t v_t^T,      o_t = S_t^T q_t (+ skip * v_t)            S: [dim x vdim], 32-bit
 // with a decay a_t and an input scale b_t that are scalars a (token, head).  Three mixers are this with other gates:
-//   * retention: a a constant of the head, b = 1;
+//   * retention: a a constant of the head, b = 1 (with q, k and v through SiLU first: lightning attention);
 //   * the matrix memory with exponential gates: a = exp(f + m_(t-1) - m_t), b = exp(i - m_t) under a running maximum
 //     m_t = max(f + m_(t-1), i); its normaliser n_t = a n_(t-1) + b k_t is the same recurrence with a value that is
 //     always 1, carried here as one more column of S, whose output is n_t . q_t;
@@ -329,6 +329,7 @@ struct ScanArgs {
     const int* cu_tokens; const int* state_slots;
     int H, dim, vdim, P, cols;                                    // cols: columns of S a block (LS_THREADS / P)
     float q_scale, k_scale;
+    int act;                                                      // IA_ACT_SILU: q, k and v go through it ahead of everything else (0: as they are)
     int wide;                                                     // the matrices' rows start at multiples of 16 bytes
     int q_vec, k_vec;                                             // so do the heads' rows of q and k, and dim is a multiple of a 16-byte load
     int stage;                                                    // tokens whose operands a block holds in shared memory at a time
@@ -336,6 +337,8 @@ struct ScanArgs {
     float* chunk_s;                                               // [seqs][max_chunks][H][vt][dim]
     float* chunk_a;                                               // [seqs][max_chunks][H]
 };
+
+__device__ __forceinline__ float ls_act(float v, int act) { return act == IA_ACT_SILU ? v / (1.0f + expf(-v)) : v; }
 
 template <typename T, int MODE, int P>
 __global__ __launch_bounds__(LS_THREADS) void linear_scan_kernel(const ScanArgs a) {
@@ -388,12 +391,12 @@ __global__ __launch_bounds__(LS_THREADS) void linear_scan_kernel(const ScanArgs 
         __syncthreads();                                          // (the stage before is used up)
         for (int e = threadIdx.x; e < nt * dimp; e += LS_THREADS) {
             const int tt = e / dimp, i = e - tt * dimp;
-            q_s[e] = i < a.dim ? ld(q + (long long)(t0 + tt) * a.q_ld + i) * a.q_scale : 0.f;
-            if (MODE != LS_CARRY) k_s[e] = i < a.dim ? ld(k + (long long)(t0 + tt) * a.k_ld + i) * a.k_scale : 0.f;
+            q_s[e] = i < a.dim ? ls_act(ld(q + (long long)(t0 + tt) * a.q_ld + i), a.act) * a.q_scale : 0.f;
+            if (MODE != LS_CARRY) k_s[e] = i < a.dim ? ls_act(ld(k + (long long)(t0 + tt) * a.k_ld + i), a.act) * a.k_scale : 0.f;
         }
         for (int e = threadIdx.x; e < nt * a.cols; e += LS_THREADS) {
             const int tt = e / a.cols, jv = j0 + e - tt * a.cols;
-            if (MODE != LS_CARRY) v_s[e] = jv < a.vdim ? ld(v + (long long)(t0 + tt) * a.v_ld + jv) : 1.f;
+            if (MODE != LS_CARRY) v_s[e] = jv < a.vdim ? ls_act(ld(v + (long long)(t0 + tt) * a.v_ld + jv), a.act) : 1.f;
             // (CARRY: what the chunk's own walk left at the places this block adds to, so that no load stands in the walk)
             else v_s[e] = jv < a.vdim ? a.out[((long long)(t0 + tt) * a.H + h) * a.vdim + jv]
                                       : jv < vt ? a.den[(long long)(t0 + tt) * a.H + h] : 0.f;
@@ -452,7 +455,7 @@ __global__ __launch_bounds__(LS_THREADS) void linear_scan_kernel(const ScanArgs 
 typedef float ls_f32x4 __attribute__((ext_vector_type(4)));
 #define LC_TOKENS 64
 
-// Rows of a chunk into shared memory as 32-bit values times `scale`: dst[tt][i] = src[(first + tt) * src_ld + i] for tt <
+// Rows of a chunk into shared memory as 32-bit values times `scale`: dst[tt][i] = act(src[(first + tt) * src_ld + i]) for tt <
 // nt and i < dim, zeros up to 64 rows and k4 columns.  `vec`: 16-byte loads (the rows start at multiples of 16 bytes and
 // dim is a multiple of what a load holds); every load of a thread is asked for before its first store.
 __device__ __forceinline__ void ls_load16(const float* p, float (&v)[8], int& n) {
@@ -463,7 +466,7 @@ __device__ __forceinline__ void ls_load16(const bf16_t* p, float (&v)[8], int& n
 
 template <typename T>
 __device__ __forceinline__ void stage_rows(float* __restrict__ dst, int ld_s, const T* __restrict__ src, long long src_ld,
-                                           int first, int nt, int dim, int k4, float scale, bool vec) {
+                                           int first, int nt, int dim, int k4, float scale, bool vec, int act) {
     constexpr int E = 16 / (int)sizeof(T);                // elements a load
     if (vec) {
         const int per_row = dim / E;                       // (k4 == dim here)
@@ -486,7 +489,7 @@ __device__ __forceinline__ void stage_rows(float* __restrict__ dst, int ld_s, co
             const int tt = idx / per_row, piece = idx - tt * per_row;
             if (idx < total) {
 #pragma unroll
-                for (int e = 0; e < E; ++e) dst[tt * ld_s + piece * E + e] = v[it][e] * scale;
+                for (int e = 0; e < E; ++e) dst[tt * ld_s + piece * E + e] = ls_act(v[it][e], act) * scale;
             }
         }
         return;
@@ -505,7 +508,7 @@ __device__ __forceinline__ void stage_rows(float* __restrict__ dst, int ld_s, co
 #pragma unroll
         for (int ic = 0; ic < 4; ++ic) {
             const int tt = (threadIdx.x >> 5) + 8 * it, i = (threadIdx.x & 31) + 32 * ic;
-            if (i < k4) dst[tt * ld_s + i] = v[it][ic] * scale;
+            if (i < k4) dst[tt * ld_s + i] = ls_act(v[it][ic], act) * scale;
         }
 }
 #define LC_COLS 32
@@ -526,7 +529,7 @@ __global__ __launch_bounds__(256) void linear_carry_mfma_kernel(const ScanArgs a
     const int nt = end - first < a.chunk ? end - first : a.chunk;
     const int k4 = (a.dim + 3) / 4 * 4;
     const T* q = (const T*)a.q + a.q_off + (long long)(h / (a.H / a.q_heads)) * a.dim;
-    stage_rows<T>(q_s, ld_s, q, a.q_ld, first, nt, a.dim, k4, a.q_scale, a.q_vec != 0);
+    stage_rows<T>(q_s, ld_s, q, a.q_ld, first, nt, a.dim, k4, a.q_scale, a.q_vec != 0, a.act);
     // (the columns of the start's matrix lie like rows of dim entries: the same staging, 32 of them)
     const float* start = a.chunk_s + ((long long)blockIdx.z * a.H + h) * vt * a.dim;
     const int cols_here = vt - j0 < LC_COLS ? vt - j0 : LC_COLS;
@@ -626,8 +629,8 @@ __global__ __launch_bounds__(256) void linear_local_mfma_kernel(const ScanArgs a
     const T* q = (const T*)a.q + a.q_off + (long long)(h / (a.H / a.q_heads)) * a.dim;
     const T* k = (const T*)a.k + a.k_off + (long long)(h / (a.H / a.k_heads)) * a.dim;
     const T* v = (const T*)a.v + a.v_off + (long long)h * a.vdim;
-    stage_rows<T>(q_s, ld_s, q, a.q_ld, first, nt, a.dim, k4, a.q_scale, a.q_vec != 0);
-    stage_rows<T>(k_s, ld_s, k, a.k_ld, first, nt, a.dim, k4, a.k_scale, a.k_vec != 0);
+    stage_rows<T>(q_s, ld_s, q, a.q_ld, first, nt, a.dim, k4, a.q_scale, a.q_vec != 0, a.act);
+    stage_rows<T>(k_s, ld_s, k, a.k_ld, first, nt, a.dim, k4, a.k_scale, a.k_vec != 0, a.act);
     if (threadIdx.x < LC_TOKENS) {
         const int tt = threadIdx.x;
         float g = 0.f, b = 0.f;
@@ -680,7 +683,7 @@ __global__ __launch_bounds__(256) void linear_local_mfma_kernel(const ScanArgs a
 #pragma unroll
             for (int it = 0; it < 8; ++it) {
                 const int tt = (threadIdx.x >> 5) + 8 * it;
-                vv[it] = (tt < nt && j < vt) ? (j < a.vdim ? ld(v + (long long)(first + tt) * a.v_ld + j) : 1.f) : 0.f;
+                vv[it] = (tt < nt && j < vt) ? (j < a.vdim ? ls_act(ld(v + (long long)(first + tt) * a.v_ld + j), a.act) : 1.f) : 0.f;
             }
 #pragma unroll
             for (int it = 0; it < 8; ++it) v_s[((threadIdx.x >> 5) + 8 * it) * LL_V_LD + (threadIdx.x & 31)] = vv[it];
@@ -782,7 +785,7 @@ extern "C" int ia_linear_scan(float* out, float* den, float* state, long long ro
                               const void* v, long long v_ld, int v_off,
                               const float* log_a, int a_per_token, const float* b, const float* skip,
                               const int* cu_tokens, const int* state_slots, int n_seqs, int H, int dim, int vdim,
-                              float q_scale, float k_scale, int chunk, int max_q_len, float* workspace, int dtype,
+                              float q_scale, float k_scale, int act, int chunk, int max_q_len, float* workspace, int dtype,
                               hipStream_t stream) {
     IA_CHECK(n_seqs >= 0 && H > 0 && dim > 0 && vdim > 0, "linear_scan: bad sizes heads=%d dim=%d vdim=%d", H, dim, vdim);
     IA_CHECK(dim <= LS_R * IA_WAVE, "linear_scan: a key size of %d is beyond %d", dim, LS_R * IA_WAVE);
@@ -794,6 +797,7 @@ extern "C" int ia_linear_scan(float* out, float* den, float* state, long long ro
              v_off >= 0 && v_off + (long long)H * vdim <= v_ld, "linear_scan: q, k or v lie outside their rows");
     IA_CHECK(chunk >= 0 && (chunk == 0 || (workspace != nullptr && max_q_len >= 1)), "linear_scan: chunks of %d tokens need a "
              "workspace and the longest portion's length", chunk);
+    IA_CHECK(act == IA_ACT_NONE || act == IA_ACT_SILU, "linear_scan: activation %d (0 none, 1 SiLU)", act);
     if (n_seqs == 0) return 0;
     int P = 1;
     while (P * LS_R < dim) P *= 2;
@@ -805,7 +809,7 @@ extern "C" int ia_linear_scan(float* out, float* den, float* state, long long ro
     a.log_a = log_a; a.a_per_token = a_per_token; a.b = b; a.skip = skip;
     a.cu_tokens = cu_tokens; a.state_slots = state_slots;
     a.H = H; a.dim = dim; a.vdim = vdim; a.P = P; a.cols = LS_THREADS / P;
-    a.q_scale = q_scale; a.k_scale = k_scale;
+    a.q_scale = q_scale; a.k_scale = k_scale; a.act = act;
     a.chunk = chunk; a.max_chunks = chunk ? (max_q_len + chunk - 1) / chunk : 1;
     a.chunk_s = workspace;
     {

@@ -2,6 +2,7 @@
 //     x <- x + y1 (+ y2) (+ sum_k [w_k] r_k) (+ s y3)          the sub-layers' outputs, every one optional
 //     x <- x + rmsnorm(t) * w_t                                  (optional) a row that enters behind the sum, normed
 //     h  = norm(x)                                               (optional) what the next layer's sub-layers read
+//     h2 = norm'(x)                                              (optional) the same with another weight, for a second reader
 // ONE kernel does any of these three in that order: a block owns a row, the sum stays in shared memory between them,
 // every statistic is 32-bit.  y1, y2, y3 may each be a product still split along its k ([splits, n, W], 32-bit); r_k
 // are the rows of routed experts [n, top, W] (32-bit) with weights w_k or, without, added as they are; s is one
@@ -29,7 +30,8 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(
     int y2_splits, int y3_splits, long long split_stride, const float* __restrict__ y3_scale,
     const float* __restrict__ routed, const float* __restrict__ routed_w, int top, const TY* __restrict__ enter,
     const float* __restrict__ enter_w, float enter_eps, TH* __restrict__ xr, const float* __restrict__ norm_w,
-    const float* __restrict__ norm_b, float norm_eps, int center, TH* __restrict__ h, const int* __restrict__ rows, int W) {
+    const float* __restrict__ norm_b, float norm_eps, int center, TH* __restrict__ h, const float* __restrict__ norm2_w,
+    const float* __restrict__ norm2_b, TH* __restrict__ h2, const int* __restrict__ rows, int W) {
     extern __shared__ float pl_row[];            // [W]
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -83,9 +85,15 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(
     }
     const float rs = 1.0f / sqrtf(block_sum(dev, scratch) / (float)W + norm_eps);
     for (int c = threadIdx.x; c < W; c += blockDim.x) {
-        float v = (pl_row[c] - mean) * rs * norm_w[c];
+        const float unit = (pl_row[c] - mean) * rs;
+        float v = unit * norm_w[c];
         if (norm_b != nullptr) v += norm_b[c];
         st(h + (long long)r * W + c, v);
+        if (h2 != nullptr) {
+            v = unit * norm2_w[c];
+            if (norm2_b != nullptr) v += norm2_b[c];
+            st(h2 + (long long)r * W + c, v);
+        }
     }
 }
 
@@ -132,7 +140,8 @@ __global__ __launch_bounds__(1024) void parallel_step_vec_kernel(
     int y2_splits, int y3_splits, long long split_stride, const float* __restrict__ y3_scale,
     const float* __restrict__ routed, const float* __restrict__ routed_w, int top, const TY* __restrict__ enter,
     const float* __restrict__ enter_w, float enter_eps, TH* __restrict__ xr, const float* __restrict__ norm_w,
-    const float* __restrict__ norm_b, float norm_eps, int center, TH* __restrict__ h, const int* __restrict__ rows, int W) {
+    const float* __restrict__ norm_b, float norm_eps, int center, TH* __restrict__ h, const float* __restrict__ norm2_w,
+    const float* __restrict__ norm2_b, TH* __restrict__ h2, const int* __restrict__ rows, int W) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int row = rows != nullptr ? rows[r] : r;
@@ -240,6 +249,16 @@ __global__ __launch_bounds__(1024) void parallel_step_vec_kernel(
             for (int i = 0; i < 8; ++i) o[i] += wv[i];
         }
         pl_store8(h + (long long)r * W + c, o);
+        if (h2 == nullptr) continue;
+        pl_load8(norm2_w + c, wv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = (v[it][i] - mean) * rs * wv[i];
+        if (norm2_b != nullptr) {
+            pl_load8(norm2_b + c, wv);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) o[i] += wv[i];
+        }
+        pl_store8(h2 + (long long)r * W + c, o);
     }
 }
 
@@ -248,13 +267,15 @@ __global__ __launch_bounds__(1024) void parallel_step_vec_kernel(
 extern "C" int ia_parallel_step(float* x, const void* y1, const void* y2, const void* y3, int y1_splits, int y2_splits,
                                 int y3_splits, const float* y3_scale, const float* routed, const float* routed_w, int top,
                                 const void* enter, const float* enter_w, float enter_eps, void* xr, const float* norm_w,
-                                const float* norm_b, float norm_eps, int center, void* h, const int* rows, int n, int W,
+                                const float* norm_b, float norm_eps, int center, void* h, const float* norm2_w,
+                                const float* norm2_b, void* h2, const int* rows, int n, int W,
                                 int y_dtype, int h_dtype, hipStream_t stream) {
     IA_CHECK(n >= 0 && W > 0 && x != nullptr, "parallel_step: n=%d width=%d, and the stream", n, W);
     IA_CHECK((size_t)W * sizeof(float) <= 60 * 1024, "parallel_step: width %d does not fit shared memory", W);
     IA_CHECK(routed == nullptr || (top >= 1 && top <= PL_MAX_TOP), "parallel_step: up to %d routed rows a row (top=%d)", PL_MAX_TOP, top);
     IA_CHECK(enter == nullptr || enter_w != nullptr, "parallel_step: a row that enters comes with its norm's weight");
     IA_CHECK(h == nullptr || norm_w != nullptr, "parallel_step: normed rows come with the norm's weight");
+    IA_CHECK(h2 == nullptr || (h != nullptr && norm2_w != nullptr), "parallel_step: rows through a second norm go beside the first's, with its weight");
     IA_CHECK(rows == nullptr || (h != nullptr && y1 == nullptr && y2 == nullptr && y3 == nullptr && routed == nullptr &&
                                  enter == nullptr && xr == nullptr),
              "parallel_step: a row list leaves the stream alone: normed rows out, nothing added");
@@ -264,7 +285,8 @@ extern "C" int ia_parallel_step(float* x, const void* y1, const void* y2, const 
     if (n == 0) return 0;
     const long long split_stride = (long long)n * W;
     const uintptr_t ptrs = (uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2 | (uintptr_t)y3 | (uintptr_t)routed | (uintptr_t)enter |
-                           (uintptr_t)enter_w | (uintptr_t)xr | (uintptr_t)norm_w | (uintptr_t)norm_b | (uintptr_t)h;
+                           (uintptr_t)enter_w | (uintptr_t)xr | (uintptr_t)norm_w | (uintptr_t)norm_b | (uintptr_t)h |
+                           (uintptr_t)norm2_w | (uintptr_t)norm2_b | (uintptr_t)h2;
     if (W % 8 == 0 && (ptrs & 15) == 0 && W <= 8 * PL_VEC_ITERS * 1024) {
         // as many threads as the row has pieces of eight, in whole waves, a round or more each
         int vthreads = (W / 8 + 63) / 64 * 64;
@@ -274,7 +296,7 @@ extern "C" int ia_parallel_step(float* x, const void* y1, const void* y2, const 
     parallel_step_vec_kernel<TY, TH><<<n, vthreads, 0, stream>>>(x, (const TY*)y1, (const TY*)y2, (const TY*)y3, y1_splits, \
                                                                  y2_splits, y3_splits, split_stride, y3_scale, routed,      \
                                                                  routed_w, top, (const TY*)enter, enter_w, enter_eps,       \
-                                                                 (TH*)xr, norm_w, norm_b, norm_eps, center, (TH*)h, rows, W)
+                                                                 (TH*)xr, norm_w, norm_b, norm_eps, center, (TH*)h, norm2_w, norm2_b, (TH*)h2, rows, W)
         if (y_dtype == IA_F32 && h_dtype == IA_F32) { IA_LAUNCH_VEC(float, float); }
         else if (y_dtype == IA_F32) { IA_LAUNCH_VEC(float, bf16_t); }
         else if (h_dtype == IA_F32) { IA_LAUNCH_VEC(bf16_t, float); }
@@ -289,7 +311,7 @@ extern "C" int ia_parallel_step(float* x, const void* y1, const void* y2, const 
     parallel_step_kernel<TY, TH><<<n, threads, shm, stream>>>(x, (const TY*)y1, (const TY*)y2, (const TY*)y3, y1_splits,  \
                                                               y2_splits, y3_splits, split_stride, y3_scale, routed,      \
                                                               routed_w, top, (const TY*)enter, enter_w, enter_eps,       \
-                                                              (TH*)xr, norm_w, norm_b, norm_eps, center, (TH*)h, rows, W)
+                                                              (TH*)xr, norm_w, norm_b, norm_eps, center, (TH*)h, norm2_w, norm2_b, (TH*)h2, rows, W)
     if (y_dtype == IA_F32 && h_dtype == IA_F32) { IA_LAUNCH(float, float); }
     else if (y_dtype == IA_F32) { IA_LAUNCH(float, bf16_t); }
     else if (h_dtype == IA_F32) { IA_LAUNCH(bf16_t, float); }

@@ -86,10 +86,14 @@ __global__ __launch_bounds__(QK_WAVES * IA_WAVE) void qk_rope_kv_kernel(
     for (int j = rot + lane; j < d; j += IA_WAVE) st(dst + j, row[j]);
 }
 
+// A value mixed with another layer's value of the same token.
+__device__ __forceinline__ float mixed_value(float v, float with, float mix) { return fmaf(mix, with, (1.0f - mix) * v); }
+
 // The same work on rows of any layout: the projections' output holds a token's query heads from `q_off`, its key heads
 // from `k_off` and its value heads (each `dv` wide, which need not be the keys' width) from `v_off`, `ld` elements a
 // row; whatever else the row holds (a gate, say) is left alone.  `k_off` < 0 or no slots: the layer writes no cache
-// (it reads another layer's), and only the queries are formed.  One wave per (token, head).
+// (it reads another layer's), and only the queries are formed.  `v_with` (rows `vw_ld` apart, value heads side by side):
+// a value becomes (1 - v_mix) v + v_mix v_with on its way to the cache.  One wave per (token, head).
 template <typename T>
 __global__ __launch_bounds__(QK_WAVES * IA_WAVE) void qk_rope_kv_strided_kernel(
     T* __restrict__ q_out,              // [n, nq, d]
@@ -99,7 +103,7 @@ __global__ __launch_bounds__(QK_WAVES * IA_WAVE) void qk_rope_kv_strided_kernel(
     const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int* __restrict__ slots,
     int n, int ld_, int q_off, int k_off, int v_off, int nq, int nkv, int d, int dv, int rot, int interleaved,
-    int page_size, float eps, int add_one) {
+    int page_size, float eps, int add_one, const T* __restrict__ v_with, long long vw_ld, float v_mix) {
     __shared__ float buf[QK_WAVES][QK_MAX_HEAD_DIM];
     const int lane = threadIdx.x & (IA_WAVE - 1);
     const int wave = threadIdx.x / IA_WAVE;
@@ -117,7 +121,8 @@ __global__ __launch_bounds__(QK_WAVES * IA_WAVE) void qk_rope_kv_strided_kernel(
     float ss = 0.f;
     if (active) {
         for (int j = lane; j < width; j += IA_WAVE) {
-            const float v = ld(src + j);
+            float v = ld(src + j);
+            if (kind == 2 && v_with != nullptr) v = mixed_value(v, ld(v_with + (size_t)tok * vw_ld + (hh - nq - nkv) * dv + j), v_mix);
             row[j] = v;
             ss += v * v;
         }
@@ -171,7 +176,8 @@ __global__ __launch_bounds__(QKS_THREADS) void qk_rope_kv_strided_bf16_vec_kerne
     bf16_t* __restrict__ q_out, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache, const bf16_t* __restrict__ proj,
     const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int* __restrict__ slots, int n, int ld_, int q_off, int k_off, int v_off, int nq,
-    int nkv, int d, int dv, int rot, int interleaved, int page_size, float eps, int add_one, int qk_blocks) {
+    int nkv, int d, int dv, int rot, int interleaved, int page_size, float eps, int add_one, int qk_blocks,
+    const bf16_t* __restrict__ v_with, long long vw_ld, float v_mix) {
     __shared__ float rows[QKS_THREADS * 8];          // normalised features, unit after unit
     __shared__ float partial[QKS_THREADS];
     if ((int)blockIdx.x >= qk_blocks) {
@@ -180,7 +186,15 @@ __global__ __launch_bounds__(QKS_THREADS) void qk_rope_kv_strided_bf16_vec_kerne
         const long long unit = (long long)((int)blockIdx.x - qk_blocks) * upb + u;
         if (u >= upb || unit >= (long long)n * nkv) return;
         const int tok = (int)(unit / nkv), hh = (int)(unit % nkv);
-        const uint4 v = *(const uint4*)(proj + (size_t)tok * ld_ + v_off + hh * dv + t * 8);
+        uint4 v = *(const uint4*)(proj + (size_t)tok * ld_ + v_off + hh * dv + t * 8);
+        if (v_with != nullptr) {
+            const uint4 f = *(const uint4*)(v_with + (size_t)tok * vw_ld + hh * dv + t * 8);
+            auto both = [&](uint32_t a, uint32_t b) {
+                return pack_bf16x2(mixed_value(__uint_as_float(a << 16), __uint_as_float(b << 16), v_mix),
+                                   mixed_value(__uint_as_float(a & 0xffff0000u), __uint_as_float(b & 0xffff0000u), v_mix));
+            };
+            v = make_uint4(both(v.x, f.x), both(v.y, f.y), both(v.z, f.z), both(v.w, f.w));
+        }
         const int slot = slots[tok];
         const int page = slot / page_size, off = slot - page * page_size;
         bf16_t* dst = v_cache + (((size_t)page * nkv + hh) * dv + t * 8) * page_size + off;
@@ -265,7 +279,9 @@ __global__ __launch_bounds__(QKS_THREADS) void qk_rope_kv_strided_bf16_vec_kerne
 extern "C" int ia_qk_rope_kv_strided(void* q_out, void* k_cache, void* v_cache, const void* proj, const float* q_norm_w,
                                      const float* k_norm_w, const float* cos_t, const float* sin_t, const int* slots, int n,
                                      int ld_, int q_off, int k_off, int v_off, int nq, int nkv, int d, int dv, int rot,
-                                     int interleaved, int page_size, float eps, int add_one, int dtype, hipStream_t stream) {
+                                     int interleaved, int page_size, float eps, int add_one, const void* v_with,
+                                     long long vw_ld, float v_mix, int dtype, hipStream_t stream) {
+    IA_CHECK(v_with == nullptr || vw_ld >= (long long)nkv * dv, "qk_rope_kv_strided: values to mix with, rows %lld apart, of %d x %d", vw_ld, nkv, dv);
     IA_CHECK(n >= 0 && nq > 0 && nkv > 0, "qk_rope_kv_strided: bad sizes n=%d nq=%d nkv=%d", n, nq, nkv);
     IA_CHECK(d > 0 && d <= QK_MAX_HEAD_DIM && dv > 0 && dv <= QK_MAX_HEAD_DIM,
              "qk_rope_kv_strided: head sizes %d / %d are outside 1..%d", d, dv, QK_MAX_HEAD_DIM);
@@ -280,9 +296,9 @@ extern "C" int ia_qk_rope_kv_strided(void* q_out, void* k_cache, void* v_cache, 
     const long long units = (long long)n * (slots ? nq + 2 * nkv : nq);
     const unsigned grid = (unsigned)((units + QK_WAVES - 1) / QK_WAVES);
     const uintptr_t ptrs = (uintptr_t)q_out | (uintptr_t)proj | (uintptr_t)(slots ? k_cache : nullptr) | (uintptr_t)q_norm_w |
-                           (uintptr_t)k_norm_w;
+                           (uintptr_t)k_norm_w | (uintptr_t)v_with;
     if (dtype == IA_BF16 && d % 8 == 0 && dv % 8 == 0 && d / 8 <= QKS_THREADS && dv / 8 <= QKS_THREADS && ld_ % 8 == 0 &&
-        q_off % 8 == 0 && (slots == nullptr || (k_off % 8 == 0 && v_off % 8 == 0)) && (ptrs & 15) == 0) {
+        q_off % 8 == 0 && (slots == nullptr || (k_off % 8 == 0 && v_off % 8 == 0)) && (v_with == nullptr || vw_ld % 8 == 0) && (ptrs & 15) == 0) {
         const long long qk_units = (long long)n * (slots ? nq + nkv : nq);
         const int upb = QKS_THREADS / (d / 8), upb_v = QKS_THREADS / (dv / 8);
         const long long qk_blocks = (qk_units + upb - 1) / upb;
@@ -290,18 +306,19 @@ extern "C" int ia_qk_rope_kv_strided(void* q_out, void* k_cache, void* v_cache, 
         IA_CHECK(qk_blocks + v_blocks < (1ll << 31), "qk_rope_kv_strided: %d tokens are too many for one launch", n);
         qk_rope_kv_strided_bf16_vec_kernel<<<(unsigned)(qk_blocks + v_blocks), QKS_THREADS, 0, stream>>>(
             (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, (const bf16_t*)proj, q_norm_w, k_norm_w, cos_t, sin_t, slots, n,
-            ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one, (int)qk_blocks);
+            ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one, (int)qk_blocks, (const bf16_t*)v_with, vw_ld,
+            v_mix);
         IA_LAUNCH_CHECK("qk_rope_kv_strided");
         return 0;
     }
     if (dtype == IA_F32)
         qk_rope_kv_strided_kernel<float><<<grid, QK_WAVES * IA_WAVE, 0, stream>>>(
             (float*)q_out, (float*)k_cache, (float*)v_cache, (const float*)proj, q_norm_w, k_norm_w, cos_t, sin_t, slots, n,
-            ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one);
+            ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one, (const float*)v_with, vw_ld, v_mix);
     else if (dtype == IA_BF16)
         qk_rope_kv_strided_kernel<bf16_t><<<grid, QK_WAVES * IA_WAVE, 0, stream>>>(
             (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, (const bf16_t*)proj, q_norm_w, k_norm_w, cos_t, sin_t, slots,
-            n, ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one);
+            n, ld_, q_off, k_off, v_off, nq, nkv, d, dv, rot, interleaved, page_size, eps, add_one, (const bf16_t*)v_with, vw_ld, v_mix);
     else
         IA_CHECK(false, "qk_rope_kv_strided: unknown dtype %d", dtype);
     IA_LAUNCH_CHECK("qk_rope_kv_strided");

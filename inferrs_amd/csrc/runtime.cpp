@@ -94,8 +94,9 @@ struct Sequence {
 
 struct Group {
     int window;           // < 0: all keys
+    int keep_first;       // with a window: so many first positions stay as well
     PagePool pool;
-    Group(int w, int pages) : window(w), pool(pages) {}
+    Group(int w, int keep, int pages) : window(w), keep_first(keep), pool(pages) {}
 };
 
 struct Cache {
@@ -148,7 +149,7 @@ struct Cache {
             const int first_needed = std::max(0, s.length - w + 1);
             std::vector<int>& table = s.tables[g];
             const int upto = std::min(first_needed / page_size, (int)table.size());
-            for (int i = 0; i < upto; ++i)
+            for (int i = pages_for(groups[g].keep_first); i < upto; ++i)
                 if (table[i] != IAR_RELEASED) {
                     if (groups[g].pool.release(table[i])) return IAR_ERROR;
                     table[i] = IAR_RELEASED;
@@ -395,13 +396,15 @@ const char* iar_last_error(void) { return g_error; }
 int iar_abi_version(void) { return IAR_ABI_VERSION; }
 
 // ---- cache manager --------------------------------------------------------------------------
-void* iar_cache_create(int page_size, int max_seqs, int n_groups, const int* windows, const int* num_pages) {
+void* iar_cache_create(int page_size, int max_seqs, int n_groups, const int* windows, const int* keep_first, const int* num_pages) {
     if (page_size < 1) { fail(IAR_ERROR, "page_size must be >= 1, got %d", page_size); return nullptr; }
     if (max_seqs < 1) { fail(IAR_ERROR, "max_seqs must be >= 1, got %d", max_seqs); return nullptr; }
     for (int g = 0; g < n_groups; ++g)
         if (num_pages[g] < 0) { fail(IAR_ERROR, "num_pages must be >= 0, got %d", num_pages[g]); return nullptr; }
+    for (int g = 0; g < n_groups; ++g)
+        if (keep_first[g] < 0) { fail(IAR_ERROR, "keep_first must be >= 0, got %d", keep_first[g]); return nullptr; }
     Cache* c = new Cache(page_size, max_seqs);
-    for (int g = 0; g < n_groups; ++g) c->groups.emplace_back(windows[g], num_pages[g]);
+    for (int g = 0; g < n_groups; ++g) c->groups.emplace_back(windows[g], keep_first[g], num_pages[g]);
     return c;
 }
 void iar_cache_destroy(void* cache) { delete C(cache); }

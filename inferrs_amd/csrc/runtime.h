@@ -22,8 +22,8 @@ const char* iar_last_error(void);
 int iar_abi_version(void);
 
 // ---- cache manager --------------------------------------------------------------------------
-// windows[g] < 0: group g keeps every key; else only the last windows[g] positions.
-void* iar_cache_create(int page_size, int max_seqs, int n_groups, const int* windows, const int* num_pages);
+// windows[g] < 0: group g keeps every key; else only the last windows[g] positions and the first keep_first[g].
+void* iar_cache_create(int page_size, int max_seqs, int n_groups, const int* windows, const int* keep_first, const int* num_pages);
 void iar_cache_destroy(void* cache);
 int iar_cache_add_sequence(void* cache, int64_t key);              // -> state slot
 int iar_cache_free_sequence(void* cache, int64_t key);

@@ -54,6 +54,7 @@ class StepContext:
     pass_input: Any = None                  # set by the model before a stop that begins a pass of a looped range: (rows or None, vector); the block takes it
     side_rows: Any = None                   # the rows of an embedding's second table for the step's tokens, which layers take slices of
     normed: Any = None                      # (norm part, rows): the stream's rows through that norm already, left by the block before
+    first_values: Optional[torch.Tensor] = None   # the values that a layer has left for later layers to mix theirs with (rows of its own projection)
     beside: Any = None                      # (rows, offset): the product of the weights that a block has laid beside a mixer's own projection
     router_logits: Any = None               # (32-bit rows, offset): the logits of the next feed-forward's router, from a product that its matrix joined
     post_rows: Any = None                   # a 32-bit stream's rows once more in the products' precision, where a part has them already (the embedding, a block's last kernel)

@@ -16,7 +16,7 @@ _PI, _PK = POINTER(c_int), POINTER(c_int64)
 _SIGNATURES = {
     "iar_last_error": (c_char_p, []),
     "iar_abi_version": (c_int, []),
-    "iar_cache_create": (c_void_p, [c_int, c_int, c_int, _PI, _PI]),
+    "iar_cache_create": (c_void_p, [c_int, c_int, c_int, _PI, _PI, _PI]),
     "iar_cache_destroy": (None, [c_void_p]),
     "iar_cache_add_sequence": (c_int, [c_void_p, c_int64]),
     "iar_cache_free_sequence": (c_int, [c_void_p, c_int64]),

@@ -348,11 +348,15 @@ def qk_rope_kv_strided(proj: torch.Tensor, nq: int, nkv: int, d: int, dv: int, *
                        v_off: Optional[int], q_norm_w: Optional[torch.Tensor], k_norm_w: Optional[torch.Tensor], eps: float,
                        add_one: bool, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], rot: int, interleaved: bool,
                        k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], slots: Optional[torch.Tensor],
-                       page_size: int) -> torch.Tensor:
+                       page_size: int, v_with: Optional[torch.Tensor] = None, v_mix: float = 0.0) -> torch.Tensor:
     """`qk_rope_kv` on rows of any layout: a row of `proj` holds the query heads from `q_off`, the key heads from `k_off`
     and the value heads (`dv` wide each) from `v_off`, and whatever else beside them.  `k_off` None: the rows hold no keys
-    or values (a layer that reads another layer's cache).  Returns q [n, nq, d]."""
+    or values (a layer that reads another layer's cache).  `v_with` [n, nkv * dv] (rows any distance apart): another layer's
+    values of the same tokens; (1 - v_mix) v + v_mix v_with is what is cached.  Returns q [n, nq, d]."""
     _dev(proj, q_norm_w, k_norm_w, cos, sin, k_cache, v_cache, slots)
+    if v_with is not None and (not v_with.is_cuda or tuple(v_with.shape) != (proj.shape[0], nkv * dv) or v_with.dtype != proj.dtype
+                               or v_with.stride(1) != 1):
+        raise KernelError(f"qk_rope_kv_strided: values to mix with {tuple(v_with.shape)} {v_with.dtype} are no {nkv} heads of {dv}")
     _f32(q_norm_w, "q_norm weight"); _f32(k_norm_w, "k_norm weight"); _f32(cos, "cos"); _f32(sin, "sin")
     if proj.dim() != 2 or proj.stride(1) != 1:
         raise KernelError(f"qk_rope_kv_strided: the projections are 2-D rows, got {tuple(proj.shape)}")
@@ -378,7 +382,7 @@ def qk_rope_kv_strided(proj: torch.Tensor, nq: int, nkv: int, d: int, dv: int, *
         _p(q_out), _p(k_cache if slots is not None else None), _p(v_cache if slots is not None else None), _p(proj),
         _p(q_norm_w), _p(k_norm_w), _p(cos), _p(sin), _p(slots), n, ld_, q_off, -1 if k_off is None else k_off,
         -1 if v_off is None else v_off, nq, nkv, d, dv, rot, int(interleaved), page_size, ctypes.c_float(eps), int(add_one),
-        _dt(proj), _stream()))
+        _p(v_with), v_with.stride(0) if v_with is not None else 0, ctypes.c_float(v_mix), _dt(proj), _stream()))
     return q_out
 
 
@@ -400,7 +404,8 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
                       positions: torch.Tensor, token_seq: torch.Tensor, block_table: torch.Tensor,
                       *, window: Optional[int], scale: float, max_kv_len: Optional[int] = None,
                       split: Optional[bool] = None, sink: bool = False, mask_chunk: Optional[int] = None,
-                      sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      sinks: Optional[torch.Tensor] = None, keep_first: int = 0,
+                      softcap: Optional[float] = None) -> torch.Tensor:
     """q [n, nq, d] against the paged cache (values may have a width of their own: v_cache [pages, nkv, dv, page_size],
     the result is [n, nq, dv]); token i sees the keys at positions <= positions[i]
     (and > positions[i] - window) of row token_seq[i] of the table.  Any head size up to 512, any
@@ -409,7 +414,8 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     and a merge kernel (`split`; None: the kernel's own rule); the bits are the same either way.
     `sink`: the softmax's denominator holds one more term, exp(0): a key of score 0 that has no value; `sinks` [nq]
     (32-bit): the term is exp(sinks[h]) for query head h instead (not scaled).  `mask_chunk`: a token sees the keys of its
-    own chunk of that many positions only (chunks counted from position 0 of the sequence), up to itself."""
+    own chunk of that many positions only (chunks counted from position 0 of the sequence), up to itself.  `keep_first`: it
+    sees the first so many positions besides.  `softcap`: a score becomes softcap * tanh(score / softcap)."""
     _dev(q, k_cache, v_cache, positions, token_seq, block_table, sinks)
     sink = _check_sinks(sinks, sink, q.shape[1])
     _i32(positions, "positions"); _i32(token_seq, "token_seq"); _i32(block_table, "block_table")
@@ -430,7 +436,8 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     _check(lib.ia_attention_generic(
         _p(out), _p(q), _p(k_cache), _p(v_cache), _p(positions), _p(token_seq), _p(block_table), n,
         block_table.shape[1], nq, nkv, d, dv, page_size, int(window or 0), ctypes.c_float(scale), _dt(q),
-        _p(ws), max_kv_len, int(bool(sink)), int(mask_chunk or 0), _p(sinks), _stream()))
+        _p(ws), max_kv_len, int(bool(sink)), int(mask_chunk or 0), _p(sinks), int(keep_first), ctypes.c_float(softcap or 0.0),
+        _stream()))
     return out
 
 
@@ -519,13 +526,14 @@ def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
                    window: Optional[int], scale: float, splits: Optional[int] = None,
                    seqs: Optional[Tuple[int, int]] = None, tokens: Optional[Tuple[int, int]] = None,
                    out: Optional[torch.Tensor] = None, sink: bool = False, mask_chunk: Optional[int] = None,
-                   sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   sinks: Optional[torch.Tensor] = None, keep_first: int = 0, softcap: Optional[float] = None) -> torch.Tensor:
     """The matrix-core kernel: bfloat16, head sizes in steps of 16 up to 256, page sizes in steps
     of 16.  Request s owns tokens cu_tokens[s]..cu_tokens[s+1] at consecutive positions.  `seqs` =
     (first, count) and `tokens` = (first, count) restrict the call to a run of requests and their
     tokens (the whole step by default); `max_q_len` and `max_kv_len` are the largest token count of
     one of these requests in this step and their largest length after it.  `out` receives the result
-    (rows outside `tokens` are left alone).  `sink`, `sinks`, `mask_chunk`: as in `attention_generic`."""
+    (rows outside `tokens` are left alone).  `sink`, `sinks`, `mask_chunk`, `keep_first`, `softcap`: as in
+    `attention_generic`."""
     _dev(q, k_cache, v_cache, positions, cu_tokens, block_table, out, sinks)
     sink = _check_sinks(sinks, sink, q.shape[1])
     _i32(positions, "positions"); _i32(cu_tokens, "cu_tokens"); _i32(block_table, "block_table")
@@ -565,7 +573,7 @@ def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
         _p(out), _p(ws), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(cu_tokens), _p(positions),
         n, seq_begin, n_seqs, token_begin, n_tokens, max_q_len, max_kv_len, block_table.shape[1], nq, nkv, d,
         page_size, int(window or 0), ctypes.c_float(scale), splits, chunk, int(bool(sink)), int(mask_chunk or 0), _p(sinks),
-        _stream()), target)
+        int(keep_first), ctypes.c_float(softcap or 0.0), _stream()), target)
     return out
 
 

@@ -240,14 +240,17 @@ class ExpertPlan:
 
 
 def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, score: str = "sigmoid",
-          renormalize: bool = False, choice_bias: Optional[torch.Tensor] = None, gates: int = 0, plan: Optional["ExpertPlan"] = None):
+          renormalize: bool = False, choice_bias: Optional[torch.Tensor] = None, gates: int = 0, plan: Optional["ExpertPlan"] = None,
+          groups: Optional[Tuple[int, int]] = None):
     """Router logits in 32-bit (router [E, width] in the precision of h; every logit is a sum of 32-bit
     multiply-adds in an order that the width alone decides), the `top` experts by score for every row:
     (experts int32 [n, top] best first, weights float32 [n, top] = score * scale).  `choice_bias` [E] (32-bit):
     the choice goes by score + bias, the weights stay the scores.  `gates`: the last `gates` rows of `router` are no
     experts: they take no part in the choice, and the sigmoids of their logits (formed like the others, in 32-bit) come
     back as a third result, float32 [n, gates].  `plan`: an `ExpertPlan` for this step; where the kernel can (bfloat16, up to 16
-    rows and 64 outputs: one block sees every choice) it orders the pairs for the experts' products on the way."""
+    rows and 64 outputs: one block sees every choice) it orders the pairs for the experts' products on the way.
+    `groups` (count, keep): the outputs form `count` equal groups of neighbours, a group is worth the sum of its two largest scores
+    (with the bias), and only outputs of the `keep` best groups can be chosen."""
     _dev(h, router, choice_bias); _f32(choice_bias, "choice_bias")
     n, W = h.shape
     E = router.shape[0] - gates
@@ -259,6 +262,7 @@ def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, score: 
             or score not in SCORE_FUNCTIONS):
         raise KernelError(f"route: router {tuple(router.shape)} {router.dtype}, top {top}, score {score!r} (up to {MAX_EXPERTS} "
                           f"experts, top up to {MAX_TOP}, scores {sorted(SCORE_FUNCTIONS)})")
+    count, keep = _groups("route", groups, E, top)
     sel = torch.empty((n, top), dtype=torch.int32, device=h.device)
     weight = torch.empty((n, top), dtype=torch.float32, device=h.device)
     gate_out = torch.empty((n, gates), dtype=torch.float32, device=h.device) if gates else None
@@ -269,15 +273,24 @@ def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, score: 
         made = tuple(_p(x) for x in plan.parts) + (plan.experts, plan.tile)
         plan.done = True
     _check(library().ia_route(_p(sel), _p(weight), _p(h), _p(router), n, W, E, top, ctypes.c_float(scale),
-                              SCORE_FUNCTIONS[score], int(renormalize), _p(choice_bias), gates, _p(gate_out), *made, _dt(h), _stream()))
+                              SCORE_FUNCTIONS[score], int(renormalize), _p(choice_bias), gates, _p(gate_out), count, keep, *made, _dt(h), _stream()))
     return (sel, weight, gate_out) if gates else (sel, weight)
+
+
+def _groups(who: str, groups: Optional[Tuple[int, int]], outputs: int, top: int) -> Tuple[int, int]:
+    if groups is None:
+        return 0, 0
+    count, keep = groups
+    if count < 1 or outputs % count or not (1 <= keep <= count) or top > keep * (outputs // count):
+        raise KernelError(f"{who}: top {top} out of {keep} of {count} equal groups of {outputs} outputs")
+    return count, keep
 
 
 ROUTE_LOGITS_ROWS = 16        # rows of a step whose router's logits may come with another product (`route_logits`)
 
 
 def route_logits(rows: torch.Tensor, off: int, experts: int, top: int, scale: float, score: str, renormalize: bool,
-                 choice_bias: Optional[torch.Tensor], gates: int, plan: ExpertPlan):
+                 choice_bias: Optional[torch.Tensor], gates: int, plan: ExpertPlan, groups: Optional[Tuple[int, int]] = None):
     """`route` from logits that a product beside the router's matrix has left: 32-bit rows [n, ..] (up to `ROUTE_LOGITS_ROWS`),
     the experts' logits from column `off` on, those of the `gates` behind them.  The plan is made as well.  Returns
     (experts, weights, gates or None)."""
@@ -285,11 +298,12 @@ def route_logits(rows: torch.Tensor, off: int, experts: int, top: int, scale: fl
     n, ld = rows.shape
     if n > ROUTE_LOGITS_ROWS or off < 0 or off + experts + gates > ld or plan.pairs != n * top or score not in SCORE_FUNCTIONS:
         raise KernelError(f"route_logits: logits {tuple(rows.shape)} at {off} for {experts} experts and {gates} gates, a plan of {plan.pairs} pairs")
+    count, keep = _groups("route_logits", groups, experts, top)
     sel = torch.empty((n, top), dtype=torch.int32, device=rows.device)
     weight = torch.empty((n, top), dtype=torch.float32, device=rows.device)
     gate_out = torch.empty((n, gates), dtype=torch.float32, device=rows.device) if gates else None
     _check(library().ia_route_logits(_p(sel), _p(weight), _p(rows), ld, off, n, experts, top, ctypes.c_float(scale), SCORE_FUNCTIONS[score],
-                                     int(renormalize), _p(choice_bias), gates, _p(gate_out), *(_p(x) for x in plan.parts), plan.experts,
+                                     int(renormalize), _p(choice_bias), gates, _p(gate_out), count, keep, *(_p(x) for x in plan.parts), plan.experts,
                                      plan.tile, _stream()))
     plan.done = True
     return sel, weight, gate_out
@@ -473,7 +487,8 @@ def parallel_step(x: torch.Tensor, *, y1=None, y2=None, y3=None, y3_scale: Optio
                   enter: Optional[torch.Tensor] = None, enter_weight: Optional[torch.Tensor] = None, enter_eps: float = 0.0,
                   x_dtype: Optional[torch.dtype] = None, norm_weight: Optional[torch.Tensor] = None,
                   norm_bias: Optional[torch.Tensor] = None, norm_eps: float = 0.0, center: bool = True,
-                  h_dtype: Optional[torch.dtype] = None, rows: Optional[torch.Tensor] = None):
+                  h_dtype: Optional[torch.dtype] = None, rows: Optional[torch.Tensor] = None,
+                  norm2_weight: Optional[torch.Tensor] = None, norm2_bias: Optional[torch.Tensor] = None):
     """What stands between two layers around a 32-bit stream x [n, width] (changed in place) whose sub-layers all read
     one normed copy of it:
 
@@ -483,7 +498,8 @@ def parallel_step(x: torch.Tensor, *, y1=None, y2=None, y3=None, y3_scale: Optio
 
     Every line and every addend may be absent.  y1, y2, y3 may each be a product still split along its k (`Partials`).
     Returns (the new x once more in `x_dtype` or None, h in `h_dtype` or None).  `rows` (int32): only these rows go
-    through the norm; nothing is added and the stream is left as it is."""
+    through the norm; nothing is added and the stream is left as it is.  `norm2_weight`, `norm2_bias`: the same rows through a
+    second norm that differs in these alone; h is then the pair of both."""
     from . import Partials
     ys = [y1, y2, y3]
     dense = [t for t in ys + [enter] if t is not None]
@@ -494,9 +510,10 @@ def parallel_step(x: torch.Tensor, *, y1=None, y2=None, y3=None, y3_scale: Optio
         if isinstance(t, Partials):
             splits[i], ys[i] = t.parts.shape[0], t.parts
     y1, y2, y3 = ys
-    _dev(x, y1, y2, y3, y3_scale, routed, routed_weights, enter, enter_weight, norm_weight, norm_bias, rows)
+    _dev(x, y1, y2, y3, y3_scale, routed, routed_weights, enter, enter_weight, norm_weight, norm_bias, rows, norm2_weight, norm2_bias)
     for t, name in ((x, "the stream"), (y3_scale, "y3_scale"), (routed, "routed rows"), (routed_weights, "routed weights"),
-                    (enter_weight, "enter_weight"), (norm_weight, "norm weight"), (norm_bias, "norm bias")):
+                    (enter_weight, "enter_weight"), (norm_weight, "norm weight"), (norm_bias, "norm bias"), (norm2_weight, "second norm weight"),
+                    (norm2_bias, "second norm bias")):
         _f32(t, name)
     n, W = x.shape
     given = [t for t in (y1, y2, y3, enter) if t is not None]
@@ -516,9 +533,11 @@ def parallel_step(x: torch.Tensor, *, y1=None, y2=None, y3=None, y3_scale: Optio
         raise KernelError("parallel_step: a factor a row goes with y3 and has one entry a row")
     if enter is not None and (enter_weight is None or enter_weight.numel() != W):
         raise KernelError("parallel_step: a row that enters comes with its norm's weight")
-    for t in (norm_weight, norm_bias):
+    for t in (norm_weight, norm_bias, norm2_weight, norm2_bias):
         if t is not None and t.numel() != W:
             raise KernelError(f"parallel_step: the norm has {t.numel()} entries, the stream is {W} wide")
+    if norm2_weight is not None and h_dtype is None:
+        raise KernelError("parallel_step: a second norm goes with normed rows out")
     if h_dtype is not None and norm_weight is None:
         raise KernelError("parallel_step: normed rows come with the norm's weight")
     count = n
@@ -532,12 +551,13 @@ def parallel_step(x: torch.Tensor, *, y1=None, y2=None, y3=None, y3_scale: Optio
         raise KernelError("parallel_step: one precision for both outputs")
     xr = torch.empty((n, W), dtype=x_dtype, device=x.device) if x_dtype is not None else None
     h = torch.empty((count, W), dtype=h_dtype, device=x.device) if h_dtype is not None else None
+    h2 = torch.empty_like(h) if norm2_weight is not None else None
     _check(library().ia_parallel_step(
         _p(x), _p(y1), _p(y2), _p(y3), splits[0], splits[1], splits[2], _p(y3_scale), _p(routed), _p(routed_weights), top,
         _p(enter), _p(enter_weight), ctypes.c_float(enter_eps), _p(xr), _p(norm_weight), _p(norm_bias),
-        ctypes.c_float(norm_eps), int(bool(center)), _p(h), _p(rows), count, W, _dt(given[0]) if given else 0,
+        ctypes.c_float(norm_eps), int(bool(center)), _p(h), _p(norm2_weight), _p(norm2_bias), _p(h2), _p(rows), count, W, _dt(given[0]) if given else 0,
         _DT[out_dtype] if out_dtype is not None else 0, _stream()))
-    return xr, h
+    return xr, h if h2 is None else (h, h2)
 
 
 def gate_rows(g: torch.Tensor, e: torch.Tensor, e_off: int, activation: str = "gelu_tanh") -> torch.Tensor:

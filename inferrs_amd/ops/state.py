@@ -138,12 +138,13 @@ def linear_scan(*, q: torch.Tensor, q_off: int, q_heads: int, k: torch.Tensor, k
                 cu_tokens: torch.Tensor, state_slots: torch.Tensor, log_a: Optional[torch.Tensor] = None,
                 decay: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None,
                 skip: Optional[torch.Tensor] = None, q_scale: float = 1.0, k_scale: float = 1.0,
-                normaliser: bool = False, max_q_len: int = 0, chunk: Optional[int] = None):
+                normaliser: bool = False, max_q_len: int = 0, chunk: Optional[int] = None, act: int = 0):
     """The recurrence S <- a S + b k v^T, o = S^T q (+ skip v) over each request's tokens, from and into the
     [heads, vdim (+ 1), dim] floats at `s_off` of its state row.  q, k, v are 2-D rows of one precision; head h reads
     q[:, q_off + (h // (heads / q_heads)) * dim ...], likewise k, and v[:, v_off + h * vdim ...].  The decay is `log_a`
     [n, heads] (logarithms, a (token, head)) or `decay` [heads] (constants); `b` [n, heads] or 1.  `normaliser`: S has
     one more column whose value is always 1; returns (o, that column's output [n, heads]).  o is 32-bit [n, heads * vdim].
+    `act` ACT_SILU: q, k and v are silu of what the rows hold.
     `max_q_len`: an upper bound of the tokens a request brings (0: unknown, the step's tokens).  `chunk`: 0 walks every
     request's tokens in order; a number cuts portions into chunks of that many tokens that run side by side (three
     kernels: each chunk from nothing, the chunks' matrices in order, what each chunk's start contributes; for keys of
@@ -181,7 +182,7 @@ def linear_scan(*, q: torch.Tensor, q_off: int, q_heads: int, k: torch.Tensor, k
     _check(lib.ia_linear_scan(
         _p(out), _p(den), _p(state), row, s_off, _p(q), q.shape[1], q_off, q_heads, _p(k), k.shape[1], k_off, k_heads,
         _p(v), v.shape[1], v_off, _p(a), int(log_a is not None), _p(b), _p(skip), _p(cu_tokens), _p(state_slots),
-        n_seqs, heads, dim, vdim, ctypes.c_float(q_scale), ctypes.c_float(k_scale), chunk, longest, _p(work), _dt(q), _stream()))
+        n_seqs, heads, dim, vdim, ctypes.c_float(q_scale), ctypes.c_float(k_scale), act, chunk, longest, _p(work), _dt(q), _stream()))
     return (out, den) if normaliser else out
 
 

@@ -19,7 +19,9 @@ go through the kernels that take rows of any layout.  Further still: a mask of c
 a query sees the keys of its own chunk of that many positions, up to itself; every attention kernel takes it beside the
 window), one gate value a head instead of one a feature (`gate_per_head`), and q and k at unit root mean square a head
 without a learned weight (`qk_unit_norm`: the norm kernels run with a weight of ones; a turn by position keeps a head's
-sum of squares, so it does not matter on which side of the turn the norm stands).
+sum of squares, so it does not matter on which side of the turn the norm stands).  And: first positions that a query sees beside
+its window (`keep_first`: the cache keeps their pages), scores capped by a tanh (`softcap`), and values mixed with those that
+an earlier layer left for the same tokens (`v_mix`: "first" leaves them, "mix" caches (1 - l) v + l v_first).
 """
 from __future__ import annotations
 
@@ -70,6 +72,8 @@ class Attention(Mixer):
             t["v_proj.bias"] = TensorSpec((spec.n_kv_heads * spec.value_dim,))
         if spec.o_bias:
             t["o_proj.bias"] = TensorSpec((spec.hidden,))
+        if spec.v_mix == "mix":
+            t["v_mix"] = TensorSpec((), "matrix")
         return t
 
     @classmethod
@@ -77,7 +81,7 @@ class Attention(Mixer):
         if not spec.own_kv:
             return None
         return PagedKV(spec.n_kv_heads, spec.head_dim, spec.kept_window,
-                       v_head_dim=spec.value_dim if spec.value_dim != spec.head_dim else None)
+                       v_head_dim=spec.value_dim if spec.value_dim != spec.head_dim else None, keep_first=spec.keep_first)
 
     def __init__(self, spec: AttentionSpec, tensors: Dict[str, torch.Tensor], dtype, device):
         if spec.n_heads % spec.n_kv_heads:
@@ -101,13 +105,19 @@ class Attention(Mixer):
             raise SpecError(f"attention: v_head_dim {spec.value_dim} is outside 1..512, the range of the attention kernels")
         if spec.values_from_keys and (spec.value_dim != spec.head_dim or not spec.own_kv):
             raise SpecError("attention: values that are the keys have the keys' width and a key projection to come from")
+        if spec.keep_first < 0 or (spec.keep_first and spec.kept_window is None):
+            raise SpecError(f"attention: keep_first {spec.keep_first} goes with a window (of this layer and of every reader)")
+        if spec.softcap is not None and not spec.softcap > 0.0:
+            raise SpecError(f"attention: softcap {spec.softcap} must be positive")
+        if spec.v_mix not in (None, "first", "mix") or (spec.v_mix and not spec.own_kv):
+            raise SpecError(f"attention: v_mix {spec.v_mix!r} is 'first' or 'mix', in a layer with values of its own")
         self.spec = spec
         named = dict(spec.names or ())
         tensors = {k: tensors[named.get(k, k)] for k in self._tensors(spec) if named.get(k, k) in tensors}
         # rows of the plain layout [q | k | v], heads of one width, go through the kernels made for it; everything else
         # (a gate in the rows, values of another width, no keys at all) through those that take any layout
         self.plain = (spec.own_kv and not spec.gate and spec.value_dim == spec.head_dim and not spec.mask_chunk
-                      and not spec.qk_unit_norm)
+                      and not spec.qk_unit_norm and not spec.keep_first and spec.softcap is None and spec.v_mix is None)
         if not self.plain:
             self._init_general(spec, tensors, dtype, device)
             return
@@ -130,6 +140,7 @@ class Attention(Mixer):
             raise SpecError("attention: a rotation law that scales cos and sin is not taken by this mixer's kernels")
 
     def _init_general(self, spec: AttentionSpec, tensors, dtype, device):
+        self.v_mix = float(tensors["v_mix"]) if spec.v_mix == "mix" else 0.0
         H, G, d, dv = spec.n_heads, spec.n_kv_heads, spec.head_dim, spec.value_dim
         stacked, at = [tensors["q_proj.weight"]], H * d
         biases = [tensors["q_proj.bias"]] if spec.qkv_bias else None
@@ -176,11 +187,20 @@ class Attention(Mixer):
         table = ctx.position_table(self.position)
         cos, sin = table if table is not None else (None, None)
         writes = cache.writable and s.own_kv
+        v_with = None
+        if s.v_mix is not None:
+            values = proj[:, self.v_off:self.v_off + G * dv]
+            if s.v_mix == "first":
+                ctx.first_values = values
+            else:
+                v_with = ctx.first_values
+                if v_with is None:
+                    raise SpecError("attention: values are mixed with those of an earlier layer of the same step, and none has left any")
         q = ops.qk_rope_kv_strided(
             proj, H, G, d, dv, q_off=self.q_off, k_off=self.k_off if writes else None, v_off=self.v_off,
             q_norm_w=self.q_norm_w, k_norm_w=self.k_norm_w, eps=self.norm_eps, add_one=self.norm_add_one, cos=cos, sin=sin,
             rot=self.position.rot_dim, interleaved=self.position.interleaved, k_cache=cache.k, v_cache=cache.v,
-            slots=group.slots if writes else None, page_size=group.page_size)
+            slots=group.slots if writes else None, page_size=group.page_size, v_with=v_with, v_mix=self.v_mix)
         a = self._attend(ctx, q, cache, group)
         joined = a.view(a.shape[0], H * dv)
         if s.gate:
@@ -194,7 +214,8 @@ class Attention(Mixer):
     def attend(s: AttentionSpec, ctx, q, cache, group):
         """The paged attention of the step's queries: the matrix cores where they take the sizes, else the plain kernel."""
         if ops.attention_mfma_fits(q.dtype, s.head_dim, group.page_size, s.value_dim):
-            common = dict(window=s.window, scale=s.softmax_scale, sink=s.sink, mask_chunk=s.mask_chunk)
+            common = dict(window=s.window, scale=s.softmax_scale, sink=s.sink, mask_chunk=s.mask_chunk,
+                          keep_first=s.keep_first, softcap=s.softcap)
             if 0 < ctx.n_single < ctx.n_seqs:
                 # single tokens (decode) and portions of prompts want different launches: the first
                 # split their long key ranges between waves, the second have columns enough
@@ -210,7 +231,7 @@ class Attention(Mixer):
                                       max_q_len=ctx.max_q_len, max_kv_len=ctx.max_kv_len, **common)
         return ops.attention_generic(q, cache.k, cache.v, ctx.positions, ctx.token_seq, group.block_table,
                                      window=s.window, scale=s.softmax_scale, max_kv_len=ctx.max_kv_len, sink=s.sink,
-                                     mask_chunk=s.mask_chunk)
+                                     mask_chunk=s.mask_chunk, keep_first=s.keep_first, softcap=s.softcap)
 
     def load_notes(self, page_size: int):
         """What the log should say once when a model with this part is set up: a decode step that cannot take the

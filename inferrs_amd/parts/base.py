@@ -36,7 +36,8 @@ from ..weights.loader import TensorSpec
 
 @dataclass(frozen=True)
 class PagedKV:
-    """Keys and values of every cached position, in pages; `window` keeps only the last ones.
+    """Keys and values of every cached position, in pages; `window` keeps only the last ones (and `keep_first` the first so
+    many beside them).
     `head_dim` is the width of a key; values have `v_head_dim` (None: the same).  `values=False`:
     one array a layer, the keys' (a mixer that caches a single row a position, a latent one say, from
     which it forms what it needs).  `value_layout`: how a page holds its values: "transposed"
@@ -48,8 +49,11 @@ class PagedKV:
     v_head_dim: Optional[int] = None
     values: bool = True
     value_layout: str = "transposed"
+    keep_first: int = 0
 
     def __post_init__(self):
+        if self.keep_first < 0 or (self.keep_first and self.window is None):
+            raise ValueError(f"PagedKV: keep_first {self.keep_first} goes with a window and is >= 0")
         if self.value_layout not in ("transposed", "rows"):
             raise ValueError(f"PagedKV: value_layout {self.value_layout!r} is neither 'transposed' nor 'rows'")
 

@@ -14,7 +14,7 @@ feed-forward of the experts' form that runs for every token (`ClampedMlp`; its o
 behind a sigmoid gate a token with `shared_gate` (its row stands behind the router's in one matrix, so that the gate is
 formed like a router's logit: `RoutedRows.extra_scale`); `weight_on_input`, a chosen expert runs on weight * h and its
 output counts as it is (`RoutedRows.weights` is None then); `activation` "silu", experts without limits,
-W_down (silu(W_gate h) * (W_up h))."""
+W_down (silu(W_gate h) * (W_up h)); `groups`, a choice among the experts of the best groups only."""
 from __future__ import annotations
 
 from typing import Dict
@@ -79,6 +79,10 @@ class RoutedExperts(FeedForward):
                             f"input on (up to {ops.mix.MAX_TOP} of {ops.mix.MAX_EXPERTS})")
         if spec.score not in ops.mix.SCORE_FUNCTIONS:
             raise SpecError(f"routed_experts: score {spec.score!r} has no kernel (known: {sorted(ops.mix.SCORE_FUNCTIONS)})")
+        if spec.groups is not None:
+            count, keep = spec.groups
+            if count < 1 or outputs % count or not (1 <= keep <= count) or spec.top > keep * (outputs // count):
+                raise SpecError(f"routed_experts: top {spec.top} out of {keep} of {count} equal groups of {outputs} outputs")
         if spec.activation not in ops.mix.EXPERT_ACTIVATIONS:
             raise SpecError(f"routed_experts: activation {spec.activation!r} has no kernel (known: {sorted(ops.mix.EXPERT_ACTIVATIONS)})")
         self.spec = spec
@@ -119,11 +123,12 @@ class RoutedExperts(FeedForward):
         if logits is not None:                       # (a block has laid the router's matrix beside one of its own)
             ctx.router_logits = None
             sel, weights, gate = ops.mix.route_logits(logits[0], logits[1], s.experts + s.identity, s.top, s.scale, s.score, s.renormalize,
-                                                      self.correction, int(s.shared_gate), plan)
+                                                      self.correction, int(s.shared_gate), plan, groups=s.groups)
         elif s.shared_gate:
-            sel, weights, gate = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, gates=1, plan=plan)
+            sel, weights, gate = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, gates=1, plan=plan,
+                                           groups=s.groups)
         else:
-            sel, weights = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, plan=plan)
+            sel, weights = ops.route(h, self.router, s.top, s.scale, s.score, s.renormalize, self.correction, plan=plan, groups=s.groups)
         rows = ops.experts_forward(h, sel, self.gate_up, self.down, s.limit, s.alpha,
                                    ff=s.intermediate if self.tiled else None,
                                    in_weight=weights if s.weight_on_input else None, activation=s.activation, plan=plan)

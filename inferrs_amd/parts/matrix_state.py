@@ -2,10 +2,12 @@
 
     S_t = a_t S_(t-1) + b_t k_t v_t^T,      o_t = S_t^T q_t
 
-with a decay a_t and an input scale b_t that are scalars a (token, head).  "retention" has a constant decay a head;
+with a decay a_t and an input scale b_t that are scalars a (token, head).  "retention" has a constant decay a head, and so
+has "lightning" (Qin et al., "Lightning Attention-2: A Free Lunch for Handling Unlimited Sequence Lengths in Large Language
+Models"), whose q, k and v pass SiLU and whose heads are normed together;
 "mlstm" (the matrix memory of the xLSTM, Beck et al., "xLSTM: Extended Long Short-Term Memory") has exponential gates
 under a running maximum and a normaliser; "mamba2" (Dao and Gu, "Transformers are SSMs") is a selective state space behind
-a short convolution.  All three run on the same recurrence kernel (`ops.linear_scan`) and the same closing kernel
+a short convolution.  All of them run on the same recurrence kernel (`ops.linear_scan`) and the same closing kernel
 (`ops.group_norm_gate`: a norm a group of features and a gate); their gates have kernels of their own.  "side_by_side"
 runs two mixers on the same input and hands both outputs, with their weights, to the kernel that adds them to the stream.
 
@@ -19,7 +21,7 @@ from typing import Dict
 import torch
 
 from .. import ops
-from ..config.spec import MatrixMemorySpec, RetentionSpec, SideBySideSpec, SpecError, StateSpaceSpec
+from ..config.spec import LightningSpec, MatrixMemorySpec, RetentionSpec, SideBySideSpec, SpecError, StateSpaceSpec
 from ..weights.loader import TensorSpec
 from .base import FixedState, Mixer, PagedAndState, PagedKV, part_class, register_mixer
 from .block import sub_tensors
@@ -33,6 +35,11 @@ def _f32(t: torch.Tensor, device) -> torch.Tensor:
 def _check_dim(kind: str, dim: int) -> None:
     if not (1 <= dim <= ops.state.SCAN_MAX_DIM):
         raise SpecError(f"{kind}: a key size of {dim} is outside 1..{ops.state.SCAN_MAX_DIM}, the range of the recurrence kernel")
+
+
+def _check_decay(kind: str, spec) -> None:
+    if len(spec.decay) != spec.n_heads or any(not (0.0 <= d <= 1.0) for d in spec.decay):
+        raise SpecError(f"{kind}: one decay in 0..1 for each of the {spec.n_heads} heads, got {list(spec.decay)}")
 
 
 @register_mixer("retention")
@@ -51,8 +58,7 @@ class Retention(Mixer):
 
     def __init__(self, spec: RetentionSpec, tensors: Dict[str, torch.Tensor], dtype, device):
         _check_dim("retention", spec.head_dim)
-        if len(spec.decay) != spec.n_heads or any(not (0.0 <= d <= 1.0) for d in spec.decay):
-            raise SpecError(f"retention: one decay in 0..1 for each of the {spec.n_heads} heads, got {list(spec.decay)}")
+        _check_decay("retention", spec)
         self.spec = spec
         self.proj = Linear([tensors["q"], tensors["k"], tensors["v"], tensors["g"]], dtype, device)
         self.o = Linear([tensors["o"]], dtype, device)
@@ -68,6 +74,47 @@ class Retention(Mixer):
                             k_scale=s.head_dim ** -0.5)
         y = ops.group_norm_gate(o, group=s.v_dim, head=s.v_dim, eps=s.norm_eps, out_dtype=proj.dtype, gate=proj,
                                 gate_off=2 * qk + vv, act=ops.state.ACT_SILU)
+        return self.o(y)
+
+
+@register_mixer("lightning")
+class Lightning(Mixer):
+    graph_safe = True
+
+    @classmethod
+    def tensors(cls, spec: LightningSpec) -> Dict[str, TensorSpec]:
+        qk, vv = spec.n_heads * spec.head_dim, spec.n_heads * spec.v_dim
+        return {"q": TensorSpec((qk, spec.hidden)), "k": TensorSpec((qk, spec.hidden)), "v": TensorSpec((vv, spec.hidden)),
+                "g": TensorSpec((vv, spec.hidden)), "o": TensorSpec((spec.hidden, vv)), "norm": TensorSpec((vv,), "norm")}
+
+    @classmethod
+    def cache_need(cls, spec: LightningSpec):
+        floats = spec.n_heads * spec.v_dim * spec.head_dim             # the matrices [heads][v_dim][dim]
+        return FixedState((-(-floats // 4) * 4,), torch.float32)       # (rows of whole 16-byte pieces)
+
+    def __init__(self, spec: LightningSpec, tensors: Dict[str, torch.Tensor], dtype, device):
+        _check_dim("lightning", spec.head_dim)
+        _check_decay("lightning", spec)
+        self.spec = spec
+        self.proj = Linear([tensors["q"], tensors["k"], tensors["v"], tensors["g"]], dtype, device)
+        self.o = Linear([tensors["o"]], dtype, device)
+        self.norm = _f32(tensors["norm"], device)
+        self.decay = torch.tensor([float(d) for d in spec.decay], dtype=torch.float32, device=device)
+
+    def forward(self, ctx, h, cache):
+        s = self.spec
+        qk, vv = s.n_heads * s.head_dim, s.n_heads * s.v_dim
+        proj = self.proj(h)                                   # [n, q | k | v | g]
+        o = ops.linear_scan(q=proj, q_off=0, q_heads=s.n_heads, k=proj, k_off=qk, k_heads=s.n_heads, v=proj, v_off=2 * qk,
+                            heads=s.n_heads, dim=s.head_dim, vdim=s.v_dim, state=cache.state, s_off=0,
+                            cu_tokens=ctx.cu_tokens, state_slots=ctx.state_slots, decay=self.decay, max_q_len=ctx.max_q_len,
+                            act=ops.state.ACT_SILU)
+        y = ops.group_norm_gate(o, group=vv, head=s.v_dim, eps=s.norm_eps, out_dtype=proj.dtype, weight=self.norm, gate=proj,
+                                gate_off=2 * qk + vv, act=ops.state.ACT_SIGMOID)
+        if getattr(ctx, "partial_sums", False):
+            split = ops.linear_partials(y, self.o.weight)
+            if split is not None:
+                return split
         return self.o(y)
 
 

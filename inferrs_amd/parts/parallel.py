@@ -1,6 +1,7 @@
 """A layer whose two sub-layers read ONE normed copy of a residual stream kept in 32-bit, their outputs added together:
 
     h = norm(x);   x <- x + mixer(h) + ffn(h)                      (a layer may lack the feed-forward)
+    h = norm(x), h' = norm'(x);   x <- x + mixer(h) + ffn(h')      (a layer of two norms: one a sub-layer, of the same rows)
     x <- x + rmsnorm(W_proj (act(W_gate x) * e)) * w               (optional: what the token itself adds behind the sum;
                                                                     e is the layer's slice of a second embedding table's row)
 
@@ -34,15 +35,16 @@ class ParallelBlock(BlockBase):
 
     @classmethod
     def tensors(cls, spec: LayerSpec) -> Dict[str, TensorSpec]:
-        if len(spec.norms) != 1 or len(spec.norm_names) != 1:
-            raise SpecError(f"the arrangement 'parallel' has one norm, the layer names {len(spec.norms)}")
+        if len(spec.norms) not in (1, 2) or len(spec.norm_names) != len(spec.norms) or (len(spec.norms) == 2 and spec.ffn is None):
+            raise SpecError(f"the arrangement 'parallel' has one norm, or one a sub-layer; the layer names {len(spec.norms)}")
         out: Dict[str, TensorSpec] = {}
         for local, ts in part_class("mixer", spec.mixer).tensors(spec.mixer).items():
             out[spec.mixer_prefix + local] = ts
         if spec.ffn is not None:
             for local, ts in part_class("ffn", spec.ffn).tensors(spec.ffn).items():
                 out[spec.ffn_prefix + local] = ts
-        out.update(norm_tensors(spec.norm_names[0], spec.norms[0]))
+        for name, nspec in zip(spec.norm_names, spec.norms):
+            out.update(norm_tensors(name, nspec))
         side = getattr(spec.residual, "side", None)
         if side is not None:
             hidden = spec.norms[0].size
@@ -60,7 +62,8 @@ class ParallelBlock(BlockBase):
         self.ffn = None
         if spec.ffn is not None:
             self.ffn = part_class("ffn", spec.ffn)(spec.ffn, sub_tensors(tensors, spec.ffn_prefix), dtype, device)
-        self.norm = build_norm(spec.norm_names[0], spec.norms[0], tensors, dtype, device)
+        self.norms = [build_norm(name, nspec, tensors, dtype, device) for name, nspec in zip(spec.norm_names, spec.norms)]
+        self.norm = self.norms[0] if len(self.norms) == 1 else NormPair(*self.norms)
         _norm_args(self.norm)                        # (refuses a norm this arrangement's kernel does not form)
         self.first_norm = self.norm
         self.side = residual.side
@@ -75,7 +78,7 @@ class ParallelBlock(BlockBase):
     graph_safe = True
 
     def parts(self):
-        return [self, self.mixer, self.ffn, self.norm, getattr(self.mixer, "position", None),
+        return [self, self.mixer, self.ffn, *self.norms, getattr(self.mixer, "position", None),
                 *getattr(self.mixer, "parts", lambda: [])(), getattr(self.ffn, "shared", None)]
 
     # ---- the model's two ends ---------------------------------------------------------------------
@@ -103,14 +106,17 @@ class ParallelBlock(BlockBase):
         # steps of few rows: a part's last product may stay split along k (gemm_mid.hip), for `ops.parallel_step` to add up
         ctx.partial_sums = self.dtype == torch.bfloat16 and ops.MID_MIN_ROWS <= x.shape[0] <= ops.MID_MAX_ROWS
         ready = getattr(ctx, "normed", None)
-        if ready is not None and ready[0] is self.norm and ready[1].shape == x.shape:
+        if ready is not None and ready[0] is self.norm:
             h = ready[1]
         else:
             h = ops.parallel_step(x, h_dtype=self.dtype, **_norm_args(self.norm))[1]
         ctx.normed = None
+        h, h_ffn = h if isinstance(h, tuple) else (h, h)
+        if h.shape != x.shape:
+            raise SpecError(f"parallel: normed rows {tuple(h.shape)} for a stream {tuple(x.shape)}")
         adds = dict(y1=_dense(self.mixer.forward(ctx, h, cache)))
         if self.ffn is not None:
-            out = self.ffn.forward(ctx, h)
+            out = self.ffn.forward(ctx, h_ffn)
             if isinstance(out, RoutedRows):
                 if out.sel is not None:
                     raise SpecError("parallel: experts that hand their input on are not taken by this arrangement")
@@ -141,8 +147,21 @@ def _dense(out):
     return out.materialize()
 
 
+class NormPair:
+    """Two norms of the same rows, one for each sub-layer, that differ in their weights (and biases) alone."""
+
+    def __init__(self, first, second):
+        self.first, self.second = first, second
+        if getattr(first, "kind", "") != getattr(second, "kind", "") or first.eps != second.eps:
+            raise SpecError("parallel: a layer's two norms are of one kind, with one eps")
+
+
 def _norm_args(norm) -> dict:
-    """The norm at the end of `ops.parallel_step`: a layer norm with weight and bias, or a plain RMS norm."""
+    """The norm at the end of `ops.parallel_step`: a layer norm with weight and bias, or a plain RMS norm; two of them for a
+    layer whose sub-layers have a norm each."""
+    if isinstance(norm, NormPair):
+        second = _norm_args(norm.second)
+        return dict(_norm_args(norm.first), norm2_weight=second["norm_weight"], norm2_bias=second["norm_bias"])
     if getattr(norm, "add_one", False) or not hasattr(norm, "weight") or not hasattr(norm, "eps"):
         raise SpecError("parallel: the norms are layer norms with weight and bias, or plain RMS norms")
     bias = getattr(norm, "bias", None)

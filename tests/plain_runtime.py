@@ -219,7 +219,8 @@ class CacheManager:
             # The next query sits at position `length` and reads keys > length - w.
             first_needed = max(0, seq.length - w + 1)
             table = seq.tables[g.index]
-            passed = [i for i in range(min(first_needed // self.page_size, len(table))) if table[i] != RELEASED]
+            kept = self._pages_for(g.need.keep_first)         # (the first positions stay)
+            passed = [i for i in range(kept, min(first_needed // self.page_size, len(table))) if table[i] != RELEASED]
             g.pool.free([table[i] for i in passed])
             for i in passed:
                 table[i] = RELEASED

@@ -79,6 +79,25 @@ def test_a_window_gives_pages_back_once_it_has_passed_them():
     assert [g.pool.num_free for g in m.groups] == [8, 4]
 
 
+@pytest.mark.parametrize("keep_first,kept_pages", [(1, 1), (4, 1), (5, 2), (12, 3)])
+def test_a_window_keeps_the_first_positions_pages(keep_first, kept_pages):
+    m = CacheManager({0: PagedKV(2, 16, window=6, keep_first=keep_first)}, page_size=4, num_pages=12, max_seqs=1)
+    m.add_sequence("a")
+    for step in range(9):                          # portions of one to nine tokens
+        assert m.reserve("a", step + 1)
+        m.commit("a", step + 1)
+        m.check_invariants()
+    # 45 tokens: the next query reads keys 40.. and the first `keep_first`
+    table = m.sequences["a"].tables[0]
+    assert len(table) == 12
+    assert [p == RELEASED for p in table] == [kept_pages <= i < 10 for i in range(12)]
+    assert m.groups[0].pool.num_free == 10 - kept_pages
+    m.free_sequence("a")
+    assert m.groups[0].pool.num_free == 12
+    with pytest.raises(ValueError, match="keep_first"):
+        PagedKV(2, 16, keep_first=2)
+
+
 def test_state_slots_lowest_free_first():
     m = CacheManager({0: FixedState((4,))}, page_size=4, num_pages=0, max_seqs=3)
     assert [m.add_sequence(i).state_slot for i in "abc"] == [0, 1, 2]

@@ -21,7 +21,7 @@ FULL = PagedKV(2, 16)
 
 def both_caches(rng, windows=True):
     page = rng.choice([1, 3, 4, 16])
-    needs = {0: FULL, 1: PagedKV(2, 16, window=rng.choice([5, 10, 33])) if windows else FULL, 2: FULL, 3: FixedState((4,))}
+    needs = {0: FULL, 1: PagedKV(2, 16, window=rng.choice([5, 10, 33]), keep_first=rng.choice([0, 0, 1, 4, 7, 40])) if windows else FULL, 2: FULL, 3: FixedState((4,))}
     n_groups = 2 if windows else 1
     pages = [rng.randint(4, 40) for _ in range(n_groups)]
     max_seqs = rng.randint(2, 6)
@@ -238,7 +238,7 @@ def test_scheduler_takes_the_decisions_of_the_plain_one(seed):
     options = dict(max_batch_size=rng.randint(1, 6), max_tokens_per_step=rng.choice([4, 16, 64]),
                    prefill_chunk=rng.choice([None, 3, 16]), max_seq_len=rng.choice([24, 48, 4096]),
                    stop_token_ids=[rng.randrange(3, 100), rng.randrange(3, 100)], row_multiple=rng.choice([0, 4, 8, 256]))
-    needs = {0: FULL, 1: PagedKV(2, 16, window=rng.choice([6, 20]))} if seed % 2 else {0: FULL}
+    needs = {0: FULL, 1: PagedKV(2, 16, window=rng.choice([6, 20]), keep_first=rng.choice([0, 3, 9]))} if seed % 2 else {0: FULL}
     ca = CacheManager(needs, page, num_pages, max_seqs)
     cb = plain.CacheManager(needs, page, num_pages, max_seqs)
     sa, sb = Scheduler(ca, **options), plain.Scheduler(cb, **options)
