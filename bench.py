@@ -18,7 +18,7 @@ choice): `mixed16` is 16 requests with prompts of 128 to 4,096 random tokens in 
 `--decode-tokens` tokens.  Its JSON line gives tokens a second over the whole run, the prompts' and the
 decoded tokens' rates apart, and the time to a request's first token.
 
-    python bench.py --design buketar|lofudra|fisanex|ligizen|vufizen [--design-shapes 1k,2k,4k]
+    python bench.py --design buketar|lofudra|fisanex|ligizen|vufizen|lumedra [--design-shapes 1k,2k,4k]
 
 measures the Buketar design (latent attention, gated recurrences, routed experts, residual streams), the Lofudra
 design (windowed sink attention beside retention, matrix memory, state space, norms on both sides) or the Fisanex design
@@ -28,7 +28,9 @@ sizes beside the dense decoder at equal width, layers and feed-forward products 
 norm a layer that both sub-layers read, latent window attention with learned sinks beside chunked attention over caches
 that layers share, experts weighted on their inputs, a token's own input a layer) beside the Fisanex design at equal size,
 or the Vufizen design (gated, normed branches; differential attention behind a short convolution beside a matrix state that fades
-by a gate a channel; routed experts in every layer) beside the Fisanex and the Lofudra design at equal width and layers: prompts of `--prefill-tokens`
+by a gate a channel; routed experts in every layer) beside the Fisanex and the Lofudra design at equal width and layers, or the
+Lumedra design (two norms of one stream a layer; lightning attention, latent attention and capped window attention beside first
+tokens that stay, over mixed values; experts chosen inside the best groups) beside the Ligizen and the Lofudra design: prompts of `--prefill-tokens`
 tokens, decode steps at `--batch` and at batch 1 through the serving loop, and every kernel's time in one prompt and one
 decode step of both.  One JSON line; the default record above is not touched by it.
 
@@ -528,6 +530,40 @@ VUFIZEN_LIKE_KERNEL = {"branch_step": "postnorm_step", "conv_qkv": "qk_rope_kv_s
                        "attention_mfma": "attention_mfma", "gate_mul": "clamped_gate_mul", "parallel_step": "postnorm_step"}
 
 
+# ---- the Lumedra design beside the Ligizen and the Lofudra design at equal size (`--design lumedra`) --------------
+# Layer sizes in the range of real models of its kind, three layers in turn: lightning attention in heads of 128 x 128 with a
+# clamped feed-forward of 3 x width; latent attention with a cached row of 256 (latent 192 + 64 turned), heads of 64 + 64 with
+# values of 64, queries through a row of width / 2, every earlier key; attention with keys and values of 128 over a quarter as
+# many key heads, a window of 1,024 beside four first tokens, capped scores, mixed values; the last two with routed experts
+# (32 in eight groups of which four stay, 4 a token, a shared expert of twice their size).  The twins are the package's
+# closest relatives: the Ligizen design (latent and grouped attention side by side, the same experts in every other layer, one
+# norm for both sub-layers) and the Lofudra design (recurrences with a matrix state a head in every layer).
+def lumedra_shape(width: int, layers: int, vocab: int = 32768):
+    heads, ff = width // 128, 3 * width // 4 // 64 * 64
+    rec = {"type": "lightning", "mixer": {"heads": heads, "dim": 128, "vdim": 128,
+                                          "decay": [1.0 - 2.0 ** (-5 - 5 * i / max(heads - 1, 1)) for i in range(heads)]},
+           "mlp": {"kind": "dense", "ff": 3 * width, "limit": 7.0}}
+    moe = {"kind": "moe", "router": {"experts": 32, "top": 4, "scale": 2.5, "groups": {"count": 8, "keep": 4}}, "expert": {"ff": ff},
+           "shared": {"ff": 2 * ff}}
+    lat = {"type": "latent_attention", "mixer": {"heads": heads, "dim": 64, "rot_dim": 64, "vdim": 64, "q_rank": width // 2, "kv_rank": 192,
+                                                 "scale": 128 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}, "mlp": moe}
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                          "softcap": 50.0, "mask": {"size": 1024, "keep_first": 4}, "v_mix": True}, "mlp": moe}
+    pattern = [rec, lat, att]
+    return {"architecture": "Lumedra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": [pattern[i % 3] for i in range(layers)]}
+
+
+def lumedra_twins(b: dict, vocab: int = 32768) -> dict:
+    return {"ligizen": ligizen_shape(b["width"], b["layers"], vocab), "lofudra": lofudra_shape(b["width"], b["layers"], vocab)}
+
+
+LUMEDRA_LIKE_KERNEL = {"parallel_step": "parallel_step", "qk_rope_kv_strided": "qk_rope_kv_strided", "latent_prep": "latent_prep",
+                       "head_product": "head_product", "norm_slice": "norm_slice", "attention_mfma": "attention_mfma",
+                       "linear_scan": "linear_scan", "group_norm_gate": "group_norm_gate", "clamped_gate_mul": "activation",
+                       "gate_mul": "clamped_gate_mul", "experts_gate_up": "experts_gate_up", "experts_down": "experts_down",
+                       "route": "route", "route_plan": "route_plan"}
+
+
 def design_main(args) -> int:
     """Prefill and decode throughput of a design at a few layer sizes beside the dense decoder (or the designs that
     are closer to it) at equal size (random weights), and the time of every kernel of one prefill and one decode step of each."""
@@ -541,7 +577,13 @@ def design_main(args) -> int:
     records = {}
     twin_label, twin_cls, twin_vocab = "dense", Qwen3Config, "vocab_size"
     twins_of = None                              # raw -> {label: raw} where a design stands beside several others
-    if args.design == "vufizen":
+    if args.design == "lumedra":
+        from inferrs_amd.config.ligizen import LigizenConfig
+        from inferrs_amd.config.lumedra import LumedraConfig
+        shapes, shape_of, config_cls, like = FISANEX_SHAPES, lumedra_shape, LumedraConfig, LUMEDRA_LIKE_KERNEL
+        title, beside = "Lumedra", "Ligizen and Lofudra at equal width and layers"
+        twins_of, twin_classes = lumedra_twins, {"ligizen": LigizenConfig, "lofudra": LofudraConfig}
+    elif args.design == "vufizen":
         from inferrs_amd.config.vufizen import VufizenConfig
         shapes, shape_of, config_cls, like = FISANEX_SHAPES, vufizen_shape, VufizenConfig, VUFIZEN_LIKE_KERNEL
         title, beside = "Vufizen", "Fisanex and Lofudra at equal width and layers"
@@ -625,9 +667,9 @@ def main() -> int:
                     help="workloads: cut prompt portions so that a step's tokens are a multiple of this (0: off)")
     ap.add_argument("--decode-run", type=int, default=8,
                     help="decode steps that the serving loop queues on the GPU at once (1: one at a time)")
-    ap.add_argument("--design", default=None, choices=["buketar", "lofudra", "fisanex", "ligizen", "vufizen"],
+    ap.add_argument("--design", default=None, choices=["buketar", "lofudra", "fisanex", "ligizen", "vufizen", "lumedra"],
                     help="instead of the headline: prefill and decode throughput of this design at a few layer sizes "
-                         "beside the dense decoder (ligizen: beside the Fisanex design; vufizen: beside the Fisanex and the Lofudra design) "
+                         "beside the dense decoder (ligizen: beside the Fisanex design; vufizen: beside the Fisanex and the Lofudra design; lumedra: beside the Ligizen and the Lofudra design) "
                          "at equal size, with every kernel's time")
     ap.add_argument("--design-shapes", default=None, help="with --design: the sizes to run, with commas (default: all)")
     args = ap.parse_args()

@@ -134,10 +134,11 @@ class LumedraConfig:
         if i in mixers:
             v_mix = "first" if i == mixers[0] else "mix"
             first = self.raw["layers"][mixers[0]]["mixer"]
-            shape = (_int(first, "kv_heads", f"layers[{mixers[0]}].mixer"), first.get("vdim", first.get("dim")))
-            if (kv_heads, vdim) != shape:
+            # (a token's values are mixed as the projections' rows, so the rows' width is what has to agree)
+            width = first.get("kv_heads", 0) * (first.get("vdim") or first.get("dim") or 0)
+            if kv_heads * vdim != width:
                 raise ConfigError(f"config.json: '{where}' mixes its values, {kv_heads} heads of {vdim}, with those of layer "
-                                  f"{mixers[0]}, {shape[0]} heads of {shape[1]}")
+                                  f"{mixers[0]}, {width} numbers a token")
         return AttentionSpec(hidden=hidden, n_heads=heads, n_kv_heads=kv_heads, head_dim=dim, position=PositionSpec("none"),
                              scale=_num(m, "scale", where), names=ATTENTION_NAMES, v_head_dim=vdim, window=window,
                              keep_first=keep_first, softcap=softcap, v_mix=v_mix)
