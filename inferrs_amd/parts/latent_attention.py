@@ -122,4 +122,8 @@ class LatentAttention(Mixer):
         # a [n, H, D]: its first `rank` features are the mixed latent rows; through W_uv, times the gate
         joined = ops.head_product(a.view(n, H * D), self.uv, x_head=D,
                                   gate=proj if s.gate else None, g_off=self.g_off, gate_per_head=s.gate_per_head)
+        if getattr(ctx, "partial_sums", False):
+            split = ops.linear_partials(joined, self.o.weight)
+            if split is not None:
+                return split
         return self.o(joined)

@@ -89,7 +89,9 @@ CFG_E = model(83, 40, [layer(lightning(2, 150, 20, (0.8, 0.99)), moe(3, 1, 16)),
                        layer(attn(2, 1, 24, 48, 0.3, softcap=4.0, v_mix=True), moe(4, 2, 24, 1.2, (2, 2), 8)),
                        layer(lightning(4, 1, 24, (0.1, 0.6, 0.9, 0.9)), dense(8, 3.0)),
                        layer(attn(2, 2, 48, 24, 0.3, v_mix=True), moe(2, 2, 8, 2.0))])
-CONFIGS = {"A": CFG_A, "B": CFG_B, "C": CFG_C, "D": CFG_D, "E": CFG_E}
+# F: no layer that caches keys at all.
+CFG_F = model(61, 32, [layer(lightning(2, 16, 16, (0.9, 0.5)), dense(48, 0.7)), layer(lightning(1, 40, 24, (0.98,)), moe(4, 2, 16, 1.0, (2, 1)))])
+CONFIGS = {"A": CFG_A, "B": CFG_B, "C": CFG_C, "D": CFG_D, "E": CFG_E, "F": CFG_F}
 
 
 def sharpened(cfg: dict, factor: float) -> dict:

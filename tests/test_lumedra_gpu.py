@@ -35,7 +35,7 @@ pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 LENGTHS = [1, 2, 3, 17, 64, 65, 130, 300, 700]
 TOL_F32 = 2e-5
-CASES = [("A", 1.0), ("B", 1.0), ("C", 1.0), ("D", 1.0), ("E", 1.0), ("A", 4.0), ("D", 2.5)]
+CASES = [("A", 1.0), ("B", 1.0), ("C", 1.0), ("D", 1.0), ("E", 1.0), ("F", 1.0), ("A", 4.0), ("D", 2.5)]
 BOTH = pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 
 
